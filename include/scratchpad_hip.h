@@ -31,7 +31,7 @@
 extern "C" {
 #endif
 
-#define SP_ABI_VERSION 13
+#define SP_ABI_VERSION 14
 #define SP_API __attribute__((visibility("default")))
 
 typedef enum { SP_F32 = 0, SP_F16 = 1, SP_BF16 = 2, SP_FP8_E5M2 = 3 /* KV pool only */ } sp_dtype;
@@ -338,7 +338,7 @@ SP_API int sp_top_k_top_p_min_p_renorm(const float* probs, int64_t row_stride, c
  *      `epilogue` (ABI 6): 0 = out[M, N] as above.  1 = w is the merged gate|up matrix [2 N, K] of LlamaMLP
  *      (gate rows first; MergedColumnParallelLinear, linear.py:423-470) and out[M, N] = SiluAndMul of the projection
  *      (nn/layers/activation.py:21-31), bit for bit the plain call followed by sp_silu_and_mul: gate_up_proj +
- *      act_fn (nn/models/llama/llama.py:62-66) in one launch.                                      */
+ *      act_fn (nn/models/llama/llama.py:62-66) in one launch.  2 (ABI 14) = max(out, 0)^2.          */
 SP_API int sp_gemm_skinny(void* out, const void* x, const void* w, int M, int N, int K, int64_t x_stride,
                    int64_t w_stride, int64_t out_stride, int epilogue, int dtype, void* stream);
 
@@ -471,10 +471,12 @@ SP_API int sp_moe_route(int32_t* ids, float* weights, const void* x, int64_t x_s
 /* (token, expert) pairs ordered by expert: offsets [experts + 1], order[pos] = pair, place[pair] = pos */
 SP_API int sp_moe_align(int32_t* offsets, int32_t* order, int32_t* place, const int32_t* ids, int pairs, int experts,
                         void* stream);
-/* out[pos, :] = w[expert(pos)] a[row(pos)], w [experts, n, k]; row(pos) = order[pos] / row_div, or pos when order is null */
+/* out[pos, :] = w[expert(pos)] a[row(pos)], w [experts, n, k]; row(pos) = order[pos] / row_div, or pos when order is null.
+ * act (ABI 14): 0 none, 1 max(out, 0)^2 on the fp32 sum.  `experts` may be less than sp_moe_align's: the pairs of the ids
+ * behind them (outputs that have no weight) get no row written.                                                        */
 SP_API int sp_moe_grouped_gemm(void* out, const void* a, const void* w, const int32_t* offsets, const int32_t* order,
                                int row_div, int pairs, int n, int k, int experts, int64_t a_stride, int64_t out_stride,
-                               int dtype, void* stream);
+                               int act, int dtype, void* stream);
 /* out[p, f] = g * sigmoid(alpha g) * (u + 1), g = min(gu[p, f], limit), u = clamp(gu[p, ff + f], -limit, limit) */
 SP_API int sp_moe_glu(void* out, const void* gu, int64_t pairs, int ff, float limit, float alpha, int dtype, void* stream);
 /* out[t] = sum over k < top, in that order, of weights[t, k] * z[place[t * top + k]] */
@@ -484,14 +486,18 @@ SP_API int sp_moe_combine(void* out, const void* z, const int32_t* place, const 
 /* Choice of experts by softmax scores on ready fp32 logits [T, experts] (sp_small_linear_f32 makes them): s = softmax
  * over all experts; ids [T, top] = the experts with the largest s (ties: the lower index), weights [T, top] = their s
  * times scale, not renormalised.                                                                                    */
-/* renorm != 0 (ABI 13): the weights are divided by their sum - the softmax over the chosen logits only.              */
-SP_API int sp_moe_softmax_topk(int32_t* ids, float* weights, const float* logits, int64_t num_tokens, int experts, int top,
+/* renorm != 0 (ABI 13): the weights are divided by their sum - the softmax over the chosen logits only.
+ * ABI 14: logits rows of logits_stride; correction (fp32 [experts], optional): the choice is by s + correction, the weights
+ * stay s; groups > keep: only experts of the `keep` groups (of experts / groups neighbours) with the largest single choice
+ * can win; gate (fp32 [T], optional): the sigmoid of logits[t, experts], one more column of the row.                    */
+SP_API int sp_moe_softmax_topk(int32_t* ids, float* weights, float* gate, const float* logits, int64_t logits_stride,
+                               const float* correction, int64_t num_tokens, int experts, int top, int groups, int keep,
                                float scale, int renorm, void* stream);
 
 /* ---- fp32 residual stream of parallel-sublayer layers (csrc/stream_norm.hip) ------------------------------------- */
-/* x[t] = embed[ids[t]] * scale  (x fp32, embed in `dtype`) */
-SP_API int sp_embed_scale(float* x, int64_t x_stride, const void* embed, const int64_t* ids, int64_t num_tokens, int width,
-                          int64_t vocab, float scale, int dtype, void* stream);
+/* x[t] = embed[ids[t]] * scale  (x fp32, embed in `dtype`); lo (optional, ABI 14): the same row in `dtype` */
+SP_API int sp_embed_scale(float* x, int64_t x_stride, void* lo, int64_t lo_stride, const void* embed, const int64_t* ids,
+                          int64_t num_tokens, int width, int64_t vocab, float scale, int dtype, void* stream);
 /* h[t] = x[t] / sqrt(mean(x[t]^2) + eps) * weight -> out_h; hs[t] = h[t] + (h[t-1] - h[t]) * mu -> out_hs (both in
  * `dtype`, either may be null; out_hs null: a plain weighted norm, the request description is not read).  The row before
  * a step's first row is state[request slot] (zeros at a sequence's first token).                                    */
@@ -515,10 +521,14 @@ SP_API int sp_qkv_rotary_store(void* q, int64_t q_stride, const void* k, int64_t
                                void* kpool, int64_t kp_stride, void* vpool, int64_t vp_stride, const int64_t* positions,
                                const int64_t* loc, const float* freq, float mag, const float* q_bias, const float* k_bias,
                                const float* v_bias, int64_t num_tokens, int heads, int kv_heads, int dim, int vdim,
-                               int rot_dims, int adjacent, int norm_values, float eps, int qk_norm, const float* q_head_scale,
+                               int rot_dims, int adjacent, int norm_values, float eps, int qk_norm,
+                               const float* q_norm_weight, const float* k_norm_weight, const float* q_head_scale,
                                float q_temp_coef, int q_temp_every, const void* v_first, int64_t vf_stride,
                                const float* v_mix, int dtype, void* stream);
-/* (ABI 13) qk_norm != 0: q and k are divided per head by their root mean square over dim after the rotation (eps inside
+/* (ABI 14) qk_norm 2: q and k are divided by that root mean square BEFORE the rotation and multiplied with q_norm_weight /
+ * k_norm_weight (fp32 [dim], shared by the heads, optional).  v null (vdim = dim): the values are the keys as projected -
+ * with k_bias, neither normed nor rotated.                                                                              */
+/* (ABI 13) qk_norm 1: q and k are divided per head by their root mean square over dim after the rotation (eps inside
  * the root).  q_head_scale (fp32 [heads], optional) and, with q_temp_every > 0, 1 + q_temp_coef * ln(floor((position + 1) /
  * q_temp_every) + 1) multiply q afterwards.  v_first (a pool of vpool's shape and type, row stride vf_stride; optional):
  * the stored value is (1 - v_mix[0]) v + v_mix[0] v_first[loc[t]].  These forms need dim, vdim <= 256.                    */
@@ -648,6 +658,20 @@ SP_API int sp_gated_delta_scan(void* out, int64_t out_stride, const void* q, int
                                const float* decay, const float* gate, const float* norm_w, float* state,
                                int64_t state_stride, int heads, int kv_heads, int dim, int vdim, float eps, SP_SEQ_PARAMS,
                                int dtype, void* stream);
+
+/* ================================================================================================================
+ * ABI 14: post-norm layers (the stream itself is normed after every sum) whose experts may hand their input on.
+ */
+/* x = N(alpha x + scale * y) weight in place (N = division by the row's root mean square, eps inside the root; x fp32);
+ * lo (optional): the new x in `dtype`.  scale, weight fp32 [width], scale optional.
+ *   z null:  y = a
+ *   else:    y = sum over k < top, in that order, of weights[t, k] * (ids[t, k] < experts ? z[place[t * top + k]] : x[t])
+ *                + gate[t] * a[t]            (a optional; gate fp32 [T], optional: 1)
+ * a, z [rows, width] in `dtype`, z contiguous.  width <= 15360.                                                         */
+SP_API int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a_stride, const void* z, const int32_t* ids,
+                        const int32_t* place, const float* weights, const float* gate, int experts, int top,
+                        const float* scale, float alpha, const float* weight, void* lo, int64_t lo_stride,
+                        int64_t num_tokens, int width, float eps, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -121,18 +121,18 @@ SIGNATURES = {
                                    _i32, _vp]),
     "sp_moe_route": (_i32, [_vp, _vp, _vp, _i64, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
     "sp_moe_align": (_i32, [_vp, _vp, _vp, _vp, _i32, _i32, _vp]),
-    "sp_moe_grouped_gemm": (_i32, [_vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _i64, _i64, _i32, _vp]),
+    "sp_moe_grouped_gemm": (_i32, [_vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _i64, _i64, _i32, _i32, _vp]),
     "sp_moe_glu": (_i32, [_vp, _vp, _i64, _i32, _f32, _f32, _i32, _vp]),
     "sp_moe_combine": (_i32, [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _i64, _i32, _vp]),
     # ---- ABI 11
-    "sp_moe_softmax_topk": (_i32, [_vp, _vp, _vp, _i64, _i32, _i32, _f32, _i32, _vp]),
-    "sp_embed_scale": (_i32, [_vp, _i64, _vp, _vp, _i64, _i32, _i64, _f32, _i32, _vp]),
+    "sp_moe_softmax_topk": (_i32, [_vp, _vp, _vp, _vp, _i64, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "sp_embed_scale": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _i64, _i32, _i64, _f32, _i32, _vp]),
     "sp_norm_shift": (_i32, [_vp, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _i64, _i32, _f32, *_SEQ, _i32, _vp]),
     "sp_norm_save_last": (_i32, [_vp, _i64, _vp, _i64, _vp, _i32, _f32, *_SEQ, _vp]),
     "sp_stream_add": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _i64, _i32, _i32, _vp]),
     "sp_qkv_rotary_store": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _f32, _vp, _vp, _vp,
-                                   _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _f32, _i32, _vp, _f32, _i32, _vp, _i64, _vp,
-                                   _i32, _vp]),
+                                   _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _f32, _i32, _vp, _vp, _vp, _f32, _i32, _vp,
+                                   _i64, _vp, _i32, _vp]),
     "sp_pool_blocks": (_i32, [_vp, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i32, _i32, _i32, *_SEQ, _i32, _vp]),
     "sp_window_attention": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i32, _i32, _i32,
                                    _i32, _i64, _i32, _f32, _vp, _f32, _i32, _vp, _vp, _i64, _i32, *_SEQ, _i32, _vp]),
@@ -157,6 +157,9 @@ SIGNATURES = {
     "sp_lowrank_gate": (_i32, [_vp, _vp, _i64, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _vp]),
     "sp_gated_delta_scan": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _i32,
                                    _i32, _i32, _f32, *_SEQ, _i32, _vp]),
+    # ---- ABI 14
+    "sp_post_norm": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _vp, _f32, _vp, _vp, _i64, _i64, _i32,
+                            _f32, _i32, _vp]),
 }
 
 
@@ -190,7 +193,7 @@ def load() -> ctypes.CDLL:
             continue
         fn.restype = res
         fn.argtypes = args
-    if lib.sp_abi_version() != 13:
+    if lib.sp_abi_version() != 14:
         raise RuntimeError("libscratchpad_hip.so ABI version mismatch")
     _lib = lib
     return lib
@@ -942,6 +945,24 @@ def _feeds_a_measured_shape(width: int) -> bool:
     return any(k == width for (_n, k) in _LIBRARY_ROWS)
 
 
+def linear_relu_square(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """max(x @ weight.T, 0)^2: one launch where ``linear`` would take the weight-streaming kernel (the square is taken of the
+    fp32 sum), the product and the activation one after the other elsewhere"""
+    if (_SKINNY_ON and x.is_cuda and x.dim() == 2 and 0 < x.shape[0] <= SKINNY_MAX_ROWS
+            and skinny_gemm_pays(x.shape[0], weight.shape[0], x.shape[1])
+            and x.dtype in (torch.float16, torch.bfloat16) and weight.dtype == x.dtype
+            and x.shape[1] % 32 == 0 and x.stride(1) == 1 and weight.stride(1) == 1
+            and x.stride(0) % 8 == 0 and weight.stride(0) % 8 == 0
+            and x.data_ptr() % 16 == 0 and weight.data_ptr() % 16 == 0):
+        M, K = x.shape
+        N = weight.shape[0]
+        out = empty_rows(M, N, x.dtype, x.device)
+        _check(load().sp_gemm_skinny(out.data_ptr(), x.data_ptr(), weight.data_ptr(), M, N, K, x.stride(0),
+                                     weight.stride(0), out.stride(0), 2, _dt(x), _stream()), "sp_gemm_skinny(relu2)")
+        return out
+    return relu_square(linear(x, weight))
+
+
 # --------------------------------------------------------------------------- per-sequence state, latent attention, experts
 class SeqParams:
     """The header's SP_SEQ_PARAMS of one step, built once per forward (``from_forward_batch``) and handed to every kernel
@@ -1176,15 +1197,17 @@ def moe_align(ids: torch.Tensor, experts: int):
 
 
 def moe_grouped_gemm(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, pairs: int, order: Optional[torch.Tensor] = None,
-                     row_div: int = 1) -> torch.Tensor:
-    """out [pairs, N]: row pos = w[expert of pos] @ a[order[pos] // row_div] (a[pos] without order); w [E, N, K]"""
+                     row_div: int = 1, act: str = "none") -> torch.Tensor:
+    """out [pairs, N]: row pos = w[expert of pos] @ a[order[pos] // row_div] (a[pos] without order); w [E, N, K]; act
+    "relu2": max(., 0)^2 of it.  Pairs of expert numbers from E on (``offsets`` may count more experts) get no row."""
     _mat(a, "a")
     if w.dim() != 3 or not w.is_contiguous() or w.dtype != a.dtype or w.shape[2] != a.shape[1]:
         raise RuntimeError("moe_grouped_gemm: w [E, N, K] contiguous of a's dtype")
     E, N, K = w.shape
     out = torch.empty((pairs, N), dtype=a.dtype, device=a.device)
     _check(load().sp_moe_grouped_gemm(out.data_ptr(), a.data_ptr(), w.data_ptr(), offsets.data_ptr(), _ptr(order), row_div,
-                                      pairs, N, K, E, a.stride(0), out.stride(0), _dt(a), _stream()), "sp_moe_grouped_gemm")
+                                      pairs, N, K, E, a.stride(0), out.stride(0), {"none": 0, "relu2": 1}[act], _dt(a), _stream()),
+           "sp_moe_grouped_gemm")
     return out
 
 
@@ -1209,27 +1232,38 @@ def moe_combine(z: torch.Tensor, place: torch.Tensor, weights: torch.Tensor) -> 
 
 # --------------------------------------------------------------------------- fp32 stream with token shift, windowed attention, scans
 def moe_route_softmax(x: torch.Tensor, router: torch.Tensor, top: int, scale: float, bias: Optional[torch.Tensor] = None,
-                      renorm: bool = False):
-    """(ids int32 [T, top], weights fp32 [T, top]): fp32 logits router x (+ bias), the largest softmax scores, times scale;
-    ``renorm``: divided by their sum (the softmax over the chosen logits only)"""
+                      renorm: bool = False, correction: Optional[torch.Tensor] = None, groups: int = 1, keep: int = 1,
+                      gate_row: bool = False):
+    """(ids int32 [T, top], weights fp32 [T, top]): fp32 logits router x (+ bias), the largest softmax scores, times
+    scale; ``renorm``: divided by their sum (the softmax over the chosen logits only).  ``correction`` fp32 [experts] joins
+    the scores for the choice only; ``groups`` > ``keep``: only experts of the ``keep`` groups of neighbours with the largest
+    single choice compete.  ``gate_row``: the router's last row is not an expert's - the sigmoid of its logit comes back as
+    a third result, fp32 [T]."""
     logits = small_linear_f32(x, router, bias)
     T, E = logits.shape
+    E -= int(gate_row)
+    if logits.stride(1) != 1 or (correction is not None and _f32(correction, "correction").numel() != E):
+        raise RuntimeError("moe_route_softmax: correction must hold one value per expert")
+    gate = torch.empty(T, dtype=torch.float32, device=x.device) if gate_row else None
     ids = torch.empty((T, top), dtype=torch.int32, device=x.device)
     weights = torch.empty((T, top), dtype=torch.float32, device=x.device)
-    _check(load().sp_moe_softmax_topk(ids.data_ptr(), weights.data_ptr(), logits.data_ptr(), T, E, top, scale, int(renorm),
-                                      _stream()), "sp_moe_softmax_topk")
-    return ids, weights
+    _check(load().sp_moe_softmax_topk(ids.data_ptr(), weights.data_ptr(), _ptr(gate), logits.data_ptr(), logits.stride(0),
+                                      _ptr(correction), T, E, top, groups, keep, scale, int(renorm), _stream()),
+           "sp_moe_softmax_topk")
+    return (ids, weights, gate) if gate_row else (ids, weights)
 
 
-def embed_scale(embed: torch.Tensor, ids: torch.Tensor, scale: float) -> torch.Tensor:
-    """fp32 [T, W] = embed[ids] * scale"""
+def embed_scale(embed: torch.Tensor, ids: torch.Tensor, scale: float, want_lo: bool = False):
+    """fp32 [T, W] = embed[ids] * scale; ``want_lo``: (that, the same in the table's dtype)"""
     _gpu(embed, ids)
     if ids.dtype != torch.int64 or embed.dim() != 2 or not embed.is_contiguous():
         raise RuntimeError("embed_scale: int64 ids, contiguous table [vocab, width]")
     x = torch.empty((ids.shape[0], embed.shape[1]), dtype=torch.float32, device=embed.device)
-    _check(load().sp_embed_scale(x.data_ptr(), x.stride(0), embed.data_ptr(), ids.data_ptr(), ids.shape[0], embed.shape[1],
-                                 embed.shape[0], scale, _dt(embed), _stream()), "sp_embed_scale")
-    return x
+    lo = empty_rows(ids.shape[0], embed.shape[1], embed.dtype, embed.device) if want_lo else None
+    _check(load().sp_embed_scale(x.data_ptr(), x.stride(0), _ptr(lo), 0 if lo is None else lo.stride(0), embed.data_ptr(),
+                                 ids.data_ptr(), ids.shape[0], embed.shape[1], embed.shape[0], scale, _dt(embed), _stream()),
+           "sp_embed_scale")
+    return (x, lo) if want_lo else x
 
 
 def norm_shift(x: torch.Tensor, weight: torch.Tensor, eps: float, dtype: torch.dtype, mu: Optional[torch.Tensor] = None,
@@ -1271,22 +1305,31 @@ def stream_add(x: torch.Tensor, a: torch.Tensor, b: Optional[torch.Tensor] = Non
            "sp_stream_add")
 
 
-def qkv_rotary_store(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor,
+def qkv_rotary_store(q: torch.Tensor, k: torch.Tensor, v: Optional[torch.Tensor], kpool: torch.Tensor, vpool: torch.Tensor,
                      positions: torch.Tensor, loc: torch.Tensor, freq: Optional[torch.Tensor], mag: float, heads: int,
                      kv_heads: int, dim: int, vdim: int, eps: float, adjacent: bool = False, norm_values: bool = True,
                      q_bias: Optional[torch.Tensor] = None, k_bias: Optional[torch.Tensor] = None,
-                     v_bias: Optional[torch.Tensor] = None, qk_norm: bool = False, q_head_scale: Optional[torch.Tensor] = None,
+                     v_bias: Optional[torch.Tensor] = None, qk_norm: int = 0, q_norm_weight: Optional[torch.Tensor] = None,
+                     k_norm_weight: Optional[torch.Tensor] = None, q_head_scale: Optional[torch.Tensor] = None,
                      q_temp: Optional[Tuple[float, int]] = None, v_first: Optional[torch.Tensor] = None,
                      v_mix: Optional[torch.Tensor] = None) -> None:
     """q [T, heads * dim] rotated in place; k rotated, v (head-normed unless ``norm_values`` is off) into the pools' rows
     loc (views: strides are taken).  ``adjacent``: coordinate 2i pairs with 2i + 1 instead of i with i + dims / 2.  fp32
-    biases, where given, are added before the rotation / the norm.  ``qk_norm``: q and k divided per head by their root
-    mean square after the rotation; ``q_head_scale`` fp32 [heads] and ``q_temp`` = (coef, every): q times the head's number
+    biases, where given, are added before the rotation / the norm.  ``v`` None: the values are the keys as projected (with
+    their bias, neither normed nor rotated).  ``qk_norm``: q and k divided per head by their root mean square - 1: after the
+    rotation, 2: before it, then times ``q_norm_weight`` / ``k_norm_weight`` (fp32 [dim]); ``q_head_scale`` fp32 [heads] and ``q_temp`` = (coef, every): q times the head's number
     and times 1 + coef ln(floor((position + 1) / every) + 1); ``v_first`` (another layer's value pool) with ``v_mix`` (fp32,
     one number): the stored value is (1 - v_mix) v + v_mix v_first[loc]."""
     for name, t, n in (("q", q, heads * dim), ("k", k, kv_heads * dim), ("v", v, kv_heads * vdim)):
+        if t is None and name == "v":
+            if dim != vdim or norm_values or v_bias is not None or v_first is not None:
+                raise RuntimeError("qkv_rotary_store: values that are keys have the keys' width and no form of their own")
+            continue
         if _mat(t, name).shape[1] != n or t.dtype != q.dtype or t.shape[0] != q.shape[0]:
             raise RuntimeError(f"qkv_rotary_store: {name} must be [T, {n}]")
+    for name, t in (("q_norm_weight", q_norm_weight), ("k_norm_weight", k_norm_weight)):
+        if t is not None and (qk_norm != 2 or _f32(t, name).numel() != dim):
+            raise RuntimeError(f"qkv_rotary_store: {name} holds dim values and goes with qk_norm 2")
     if kpool.dtype != q.dtype or vpool.dtype != q.dtype or _mat(kpool, "kpool").shape[1] != kv_heads * dim or \
             _mat(vpool, "vpool").shape[1] != kv_heads * vdim:
         raise RuntimeError("qkv_rotary_store: pools [P, kv_heads * dim] / [P, kv_heads * vdim] of q's dtype")
@@ -1302,11 +1345,13 @@ def qkv_rotary_store(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, kpool: t
                                 v_first.dtype != vpool.dtype):
         raise RuntimeError("qkv_rotary_store: v_first must mirror vpool and come with v_mix (one fp32 number)")
     coef, every = q_temp if q_temp else (0.0, 0)
-    _check(load().sp_qkv_rotary_store(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
+    _check(load().sp_qkv_rotary_store(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), _ptr(v),
+                                      0 if v is None else v.stride(0),
                                       kpool.data_ptr(), kpool.stride(0), vpool.data_ptr(), vpool.stride(0), positions.data_ptr(),
                                       loc.data_ptr(), _ptr(freq), mag, _ptr(q_bias), _ptr(k_bias), _ptr(v_bias), q.shape[0],
                                       heads, kv_heads, dim, vdim, dims, int(adjacent), int(norm_values), eps, int(qk_norm),
-                                      _ptr(q_head_scale), float(coef), int(every), _ptr(v_first),
+                                      _ptr(q_norm_weight), _ptr(k_norm_weight), _ptr(q_head_scale), float(coef), int(every),
+                                      _ptr(v_first),
                                       0 if v_first is None else v_first.stride(0), _ptr(v_mix), _dt(q), _stream()),
            "sp_qkv_rotary_store")
 
@@ -1605,3 +1650,34 @@ def gated_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, bpre: to
                                       gate.data_ptr(), norm_w.data_ptr(), state.data_ptr(), state.stride(0), heads, kv_heads,
                                       dim, vdim, eps, *seq.args, _dt(q), _stream()), "sp_gated_delta_scan")
     return out
+
+
+# --------------------------------------------------------------------------- post-norm stream
+def post_norm(x: torch.Tensor, a: Optional[torch.Tensor], weight: torch.Tensor, eps: float, alpha: float, dtype: torch.dtype,
+              scale: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
+              place: Optional[torch.Tensor] = None, weights: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+              experts: int = 0, want_lo: bool = True) -> Optional[torch.Tensor]:
+    """x fp32 [T, W] = N(alpha x + scale * y) * weight in place; returns the new x in ``dtype`` (``want_lo``).  y = a, or with
+    a mixture's rows z [T * top, W]: y[t] = sum_k weights[t, k] (z[place[t, k]], or x[t] itself where ids[t, k] >= experts)
+    + gate[t] a[t] (a optional, gate fp32 [T] or None: 1)."""
+    _mat(x, "x"), _f32(weight, "weight")
+    T, W = x.shape
+    if x.dtype != torch.float32 or weight.numel() != W or (scale is not None and _f32(scale, "scale").numel() != W):
+        raise RuntimeError("post_norm: x fp32 [T, W], weight and scale [W]")
+    if a is not None and (_mat(a, "a").shape != (T, W) or a.dtype != dtype):
+        raise RuntimeError("post_norm: a must be [T, W] of the given dtype")
+    if z is None and (a is None or gate is not None):
+        raise RuntimeError("post_norm: a result or a mixture's rows; a gate goes with the latter")
+    top = 0
+    if z is not None:
+        top = weights.shape[1]
+        if z.dim() != 2 or not z.is_contiguous() or z.shape != (T * top, W) or z.dtype != dtype or ids.shape != (T, top) or \
+                weights.shape[0] != T or ids.dtype != torch.int32 or place.dtype != torch.int32 or place.numel() != T * top or \
+                not ids.is_contiguous() or not _f32(weights, "weights").is_contiguous() or experts <= 0 or \
+                (gate is not None and _f32(gate, "gate").numel() != T):
+            raise RuntimeError("post_norm: z [T * top, W] contiguous, ids / weights [T, top], place [T * top], gate [T]")
+    lo = empty_rows(T, W, dtype, x.device) if want_lo else None
+    _check(load().sp_post_norm(x.data_ptr(), x.stride(0), _ptr(a), 0 if a is None else a.stride(0), _ptr(z), _ptr(ids),
+                               _ptr(place), _ptr(weights), _ptr(gate), experts, top, _ptr(scale), alpha, weight.data_ptr(),
+                               _ptr(lo), 0 if lo is None else lo.stride(0), T, W, eps, _DTYPES[dtype], _stream()), "sp_post_norm")
+    return lo

@@ -540,7 +540,10 @@ class PooledWindowAttention(nn.Module):
     ``sinks``: one learned fp32 number per query head whose exponential joins the softmax's denominator (a key every query
     sees, without a value).  ``norm_values``: the cache holds every value head divided by its root mean square.  q, k, v may
     carry fp32 biases (``store``), added before the rotation.
-    ``qk_norm``: q and k are divided per head by their root mean square after the rotation.  ``head_scale``: a learned fp32
+    ``qk_norm`` "after" (or True): q and k are divided per head by their root mean square after the rotation; "before": before
+    it, and multiplied with learned fp32 weights per coordinate that the heads share (``q_norm``, ``k_norm``).
+    ``keys_as_values``: the cached value is the key as projected (bias included), neither normed nor rotated; such a layer
+    has no value projection (``store`` takes no v).  ``head_scale``: a learned fp32
     number per query head that multiplies its scores (folded into q).  ``q_temp`` = (coef, every): q of position p times
     1 + coef ln(floor((p + 1) / every) + 1).  ``softcap``: scores capped as cap tanh(score / cap).  ``weights`` = "sigmoid":
     no softmax - a visible key weighs sigmoid(score + head_bias[head]) (``head_bias`` a learned fp32 number per head), not
@@ -549,8 +552,8 @@ class PooledWindowAttention(nn.Module):
 
     def __init__(self, num_heads: int, num_kv_heads: int, dim: int, vdim: int, scaling: float, layer_id: int,
                  window: Optional[int] = None, block: Optional[int] = None, sinks: bool = False, norm_values: bool = True,
-                 qk_norm: bool = False, head_scale: bool = False, q_temp=None, softcap: float = 0.0,
-                 weights: str = "softmax", v_mix: bool = False):
+                 qk_norm=False, head_scale: bool = False, q_temp=None, softcap: float = 0.0,
+                 weights: str = "softmax", v_mix: bool = False, keys_as_values: bool = False):
         super().__init__()
         if num_heads % num_kv_heads:
             raise ValueError("query heads must be a multiple of key/value heads")
@@ -563,7 +566,13 @@ class PooledWindowAttention(nn.Module):
             raise ValueError("weights: 'softmax' or 'sigmoid' (which has no sink)")
         f32 = dict(dtype=torch.float32)
         self.sinks = nn.Parameter(torch.zeros(num_heads, **f32), requires_grad=False) if sinks else None
-        self.qk_norm, self.softcap, self.sigmoid_weights = qk_norm, float(softcap or 0.0), weights == "sigmoid"
+        if keys_as_values and (dim != vdim or norm_values or v_mix):
+            raise ValueError("values that are keys have the keys' width, no norm and no blending")
+        self.keys_as_values = keys_as_values
+        self.qk_norm = {False: 0, None: 0, True: 1, "after": 1, "before": 2}[qk_norm]
+        self.q_norm = nn.Parameter(torch.ones(dim, **f32), requires_grad=False) if self.qk_norm == 2 else None
+        self.k_norm = nn.Parameter(torch.ones(dim, **f32), requires_grad=False) if self.qk_norm == 2 else None
+        self.softcap, self.sigmoid_weights = float(softcap or 0.0), weights == "sigmoid"
         self.q_temp = (float(q_temp[0]), int(q_temp[1])) if q_temp else None
         self.head_scale = nn.Parameter(torch.ones(num_heads, **f32), requires_grad=False) if head_scale else None
         self.head_bias = nn.Parameter(torch.zeros(num_heads, **f32), requires_grad=False) if self.sigmoid_weights else None
@@ -636,6 +645,8 @@ class SequenceBackend(AttentionBackend):
                                  layer.tp_k_head_num, layer.dim, layer.vdim, eps,
                                  adjacent=bool(rotary is not None and rotary.adjacent_pairs), norm_values=layer.norm_values,
                                  q_bias=biases[0], k_bias=biases[1], v_bias=biases[2], qk_norm=layer.qk_norm,
+                                 q_norm_weight=None if layer.q_norm is None else layer.q_norm.data,
+                                 k_norm_weight=None if layer.k_norm is None else layer.k_norm.data,
                                  q_head_scale=None if layer.head_scale is None else layer.head_scale.data, q_temp=layer.q_temp,
                                  v_first=None if v_first_cache is None else pool.get_value_buffer(v_first_cache),
                                  v_mix=None if (v_first_cache is None or layer.v_mix is None) else layer.v_mix.data)

@@ -26,6 +26,7 @@
 // the activation in the PROLOGUE of the down projection, every workgroup recomputing the M x K activations it
 // streams - was built first and measured 2 x SLOWER than the two launches: 76 vs 38 us at 1 row; the exponentials
 // of all 16 lane rows of every k-step are vector work the stream cannot hide.  profiles/NOTES.md, round 4.)
+// `epilogue` = 2: out = max(product, 0)^2 on the fp32 sum, rounded once (the up projection of a squared-ReLU feed-forward).
 #include "sp_common.h"
 
 namespace sp {
@@ -72,7 +73,7 @@ __device__ __forceinline__ u32x4 ld16_nt(const void* p) { return __builtin_nonte
 template <typename Tag, int NB, int UNROLL, bool NT, int EPI>
 __global__ __launch_bounds__(kSkWaves * 64) void gemm_skinny_kernel(SkinnyArgs a) {
   typedef Elem<Tag> E;
-  static_assert(EPI == 0 || NB == 1, "the SiLU-mul epilogue pairs the two halves of one 16-row tile");
+  static_assert(EPI != 1 || NB == 1, "the SiLU-mul epilogue pairs the two halves of one 16-row tile");
   __shared__ float red[kSkWaves][NB][16 * 17];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r16 = lane & 15, q = lane >> 4;            // operand row / k-quarter of the lane
@@ -137,6 +138,10 @@ __global__ __launch_bounds__(kSkWaves * 64) void gemm_skinny_kernel(SkinnyArgs a
           E::store(a.out, (int64_t)r16 * a.out_stride + n, __fmul_rn(E::round(silu_ref(E::round(s))), E::round(su)));
       } else {
         const int n = n0 + 16 * nb + col;
+        if constexpr (EPI == 2) {
+          s = fmaxf(s, 0.f);
+          s *= s;
+        }
         if (mrow && n < a.N) E::store(a.out, (int64_t)r16 * a.out_stride + n, s);
       }
     }
@@ -156,6 +161,7 @@ static void launch_skinny(const SkinnyArgs& a, int epilogue, hipStream_t st) {
   const bool u16 = g_skinny_u16 && (a.K / 32) % (16 * kSkWaves) == 0;
   if (epilogue == 1 && u16) gemm_skinny_kernel<Tag, 1, 16, false, 1><<<dim3((a.N + 7) / 8), block, 0, st>>>(a);
   else if (epilogue == 1) gemm_skinny_kernel<Tag, 1, 8, false, 1><<<dim3((a.N + 7) / 8), block, 0, st>>>(a);
+  else if (epilogue == 2) gemm_skinny_kernel<Tag, 1, 8, false, 2><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
   else if (u16) gemm_skinny_kernel<Tag, 1, 16, false, 0><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
   else if (g_skinny_nt) gemm_skinny_kernel<Tag, 1, 8, true, 0><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
   else gemm_skinny_kernel<Tag, 1, 8, false, 0><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
@@ -165,7 +171,7 @@ static void launch_skinny(const SkinnyArgs& a, int epilogue, hipStream_t st) {
 
 extern "C" int sp_gemm_skinny(void* out, const void* x, const void* w, int M, int N, int K, int64_t x_stride,
                               int64_t w_stride, int64_t out_stride, int epilogue, int dtype, void* stream) {
-  SP_CHECK_ARG(M >= 0 && N >= 0 && K > 0 && (epilogue == 0 || epilogue == 1));
+  SP_CHECK_ARG(M >= 0 && N >= 0 && K > 0 && epilogue >= 0 && epilogue <= 2);
   if (M == 0 || N == 0) return SP_OK;
   SP_CHECK_ARG(out && x && w);
   if (M > 16 || K % 32 != 0) return SP_ERR_UNSUPPORTED;

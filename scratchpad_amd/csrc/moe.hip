@@ -1,4 +1,5 @@
-// Mixture of experts: fp32 router with sigmoid scores, a choice correction and group-limited top-k; the (token, expert)
+// Mixture of experts: fp32 routers - sigmoid scores, or softmax scores on ready logits - with a choice correction and
+// group-limited top-k; the (token, expert)
 // pairs of a step ordered by expert on the device; a grouped matrix product over that order (every expert's weights are
 // read once per row tile, fp32 accumulation); the clamped gated activation; and the weighted sum of a token's experts in
 // a fixed order, so a token's result does not depend on which other tokens share the step.
@@ -80,28 +81,50 @@ __global__ void moe_route_kernel(int32_t* ids, float* weights, const void* x, in
 }
 
 // ---- softmax scores and choice on ready fp32 logits: one wave per token ---------------------------------------------
-// s = softmax(z) over all experts; the `top` largest s win (ties: the lower index); weights = s * scale
-__global__ void moe_softmax_topk_kernel(int32_t* ids, float* weights, const float* logits, int64_t T, int E, int top,
-                                        float scale, int renorm) {
+// s = softmax(z) over all experts; choice = s + correction (s itself without one); with groups > keep only experts of the
+// `keep` groups with the largest single choice can win, whatever the others' signs; the `top` largest choices win (ties:
+// the lower index); weights = s * scale.  gate: sigmoid of the logit behind the experts' (column E of the row).
+__global__ void moe_softmax_topk_kernel(int32_t* ids, float* weights, float* gate, const float* logits, int64_t z_stride,
+                                        const float* correction, int64_t T, int E, int top, int groups, int keep, float scale,
+                                        int renorm) {
   extern __shared__ float smem[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int64_t t = (int64_t)blockIdx.x * (blockDim.x >> 6) + wave;
   if (t >= T) return;
-  float* score = smem + (size_t)wave * 2 * E;     // s[E], then the choice copy
+  float* score = smem + (size_t)wave * (2 * E + groups);     // s[E], choice[E], group score[groups]
   float* choice = score + E;
+  float* gscore = choice + E;
+  const float* z = logits + t * z_stride;
+  if (gate && lane == 0) gate[t] = 1.f / (1.f + expf(-z[E]));
   float zmax = -INFINITY;
-  for (int e = lane; e < E; e += 64) zmax = fmaxf(zmax, logits[t * E + e]);
+  for (int e = lane; e < E; e += 64) zmax = fmaxf(zmax, z[e]);
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) zmax = fmaxf(zmax, __shfl_xor(zmax, off, 64));
   float part = 0.f;
-  for (int e = lane; e < E; e += 64) part += expf(logits[t * E + e] - zmax);
+  for (int e = lane; e < E; e += 64) part += expf(z[e] - zmax);
   const float inv = 1.f / wave_sum(part);
   for (int e = lane; e < E; e += 64) {
-    const float sv = expf(logits[t * E + e] - zmax) * inv;
+    const float sv = expf(z[e] - zmax) * inv;
     score[e] = sv;
-    choice[e] = sv;
+    choice[e] = correction ? sv + correction[e] : sv;
   }
   __builtin_amdgcn_wave_barrier();
+  if (keep < groups) {
+    const int per = E / groups;
+    for (int g = lane; g < groups; g += 64) {
+      float best = -INFINITY;
+      for (int e = g * per; e < (g + 1) * per; ++e) best = fmaxf(best, choice[e]);
+      gscore[g] = best;
+    }
+    __builtin_amdgcn_wave_barrier();
+    for (int g = lane; g < groups; g += 64) {             // every lane judges its groups: ties leave the lower index in
+      int better = 0;
+      for (int o = 0; o < groups; ++o) better += (gscore[o] > gscore[g]) || (gscore[o] == gscore[g] && o < g);
+      if (better >= keep)
+        for (int e = g * per; e < (g + 1) * per; ++e) choice[e] = -INFINITY;
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
   float chosen = 0.f;                                  // lane 0: the sum of the chosen scores
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
@@ -156,14 +179,21 @@ __global__ void moe_align_kernel(int32_t* offsets, int32_t* order, int32_t* plac
 }
 
 // ---- grouped product: out[pos, n] = sum_k a[row(pos), k] * w[expert(pos), n, k] -------------------------------------
-// row(pos) = order[pos] / row_div when order is given (the token of a pair), else pos.  Tiles of 32 rows x 64 columns;
+// row(pos) = order[pos] / row_div when order is given (the token of a pair), else pos; act 1: max(out, 0)^2 instead (on the
+// fp32 sum, rounded once).  Pairs of ids from E on (outputs without a weight) are left alone.  Tiles of 32 rows x 64 columns;
 // a tile never spans two experts.  Each output element accumulates over k in the same order wherever its row sits.
 constexpr int GM = 32, GN = 64, GK = 32;
+
+__device__ __forceinline__ float gemm_act(float v, int act) {
+  if (act == 0) return v;
+  const float r = fmaxf(v, 0.f);
+  return r * r;
+}
 
 template <typename Tag>
 __global__ void __launch_bounds__(256)
 moe_grouped_gemm_kernel(void* out, const void* a, const void* w, const int32_t* offsets, const int32_t* order, int row_div,
-                        int P, int N, int K, int E, int64_t a_stride, int64_t out_stride) {
+                        int P, int N, int K, int E, int64_t a_stride, int64_t out_stride, int act) {
   typedef Elem<Tag> El;
   __shared__ float As[GK][GM + 1];
   __shared__ float Bs[GK][GN + 4];
@@ -220,7 +250,7 @@ moe_grouped_gemm_kernel(void* out, const void* a, const void* w, const int32_t* 
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) El::store(out, (int64_t)pos * out_stride + n, acc[i][j]);
+      if (n < N) El::store(out, (int64_t)pos * out_stride + n, gemm_act(acc[i][j], act));
     }
   }
 }
@@ -251,7 +281,7 @@ constexpr int QM = 128, QN = 64;
 template <typename Tag>
 __global__ void __launch_bounds__(256)
 moe_grouped_mfma_kernel(void* out, const void* a, const void* w, const int32_t* offsets, const int32_t* order, int row_div,
-                        int N, int K, int E, int64_t a_stride, int64_t out_stride) {
+                        int N, int K, int E, int64_t a_stride, int64_t out_stride, int act) {
   typedef Elem<Tag> El;
   int tile = blockIdx.x, e = 0, row0 = 0, rows_end = 0;
   for (; e < E; ++e) {
@@ -310,7 +340,7 @@ moe_grouped_mfma_kernel(void* out, const void* a, const void* w, const int32_t* 
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int n = n0 + 16 * j + 4 * q + r;
-        if (n < N) El::store(out, (int64_t)pos * out_stride + n, acc[f][j][r]);
+        if (n < N) El::store(out, (int64_t)pos * out_stride + n, gemm_act(acc[f][j][r], act));
       }
   }
 }
@@ -363,16 +393,18 @@ extern "C" int sp_moe_route(int32_t* ids, float* weights, const void* x, int64_t
   return SP_OK;
 }
 
-extern "C" int sp_moe_softmax_topk(int32_t* ids, float* weights, const float* logits, int64_t num_tokens, int experts, int top,
+extern "C" int sp_moe_softmax_topk(int32_t* ids, float* weights, float* gate, const float* logits, int64_t logits_stride,
+                                   const float* correction, int64_t num_tokens, int experts, int top, int groups, int keep,
                                    float scale, int renorm, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && experts > 0 && top > 0 && top <= experts);
+  SP_CHECK_ARG(groups >= 1 && keep >= 1 && keep <= groups && experts % groups == 0);
+  SP_CHECK_ARG((int64_t)top <= (int64_t)keep * (experts / groups));
   if (num_tokens == 0) return SP_OK;
-  SP_CHECK_ARG(ids && weights && logits);
-  const size_t lds = 4 * (size_t)(2 * experts) * sizeof(float);
+  SP_CHECK_ARG(ids && weights && logits && logits_stride >= experts + (gate ? 1 : 0));
+  const size_t lds = 4 * (size_t)(2 * experts + groups) * sizeof(float);
   if (lds > 64 * 1024) return SP_ERR_UNSUPPORTED;
-  moe_softmax_topk_kernel<<<dim3((unsigned)((num_tokens + 3) / 4)), 256, lds, (hipStream_t)stream>>>(ids, weights, logits,
-                                                                                                  num_tokens, experts, top, scale,
-                                                                                                  renorm);
+  moe_softmax_topk_kernel<<<dim3((unsigned)((num_tokens + 3) / 4)), 256, lds, (hipStream_t)stream>>>(
+      ids, weights, gate, logits, logits_stride, correction, num_tokens, experts, top, groups, keep, scale, renorm);
   SP_LAUNCH_CHECK();
   return SP_OK;
 }
@@ -389,8 +421,8 @@ extern "C" int sp_moe_align(int32_t* offsets, int32_t* order, int32_t* place, co
 
 extern "C" int sp_moe_grouped_gemm(void* out, const void* a, const void* w, const int32_t* offsets, const int32_t* order,
                                    int row_div, int pairs, int n, int k, int experts, int64_t a_stride,
-                                   int64_t out_stride, int dtype, void* stream) {
-  SP_CHECK_ARG(pairs >= 0 && n > 0 && k > 0 && experts > 0 && row_div >= 1);
+                                   int64_t out_stride, int act, int dtype, void* stream) {
+  SP_CHECK_ARG(pairs >= 0 && n > 0 && k > 0 && experts > 0 && row_div >= 1 && (act == 0 || act == 1));
   if (pairs == 0) return SP_OK;
   SP_CHECK_ARG(out && a && w && offsets && a_stride >= k && out_stride >= n);
   const bool aligned = k % 32 == 0 && a_stride % 8 == 0 && ((uintptr_t)a & 15) == 0 && ((uintptr_t)w & 15) == 0;
@@ -398,16 +430,16 @@ extern "C" int sp_moe_grouped_gemm(void* out, const void* a, const void* w, cons
     const dim3 grid((unsigned)((pairs + QM - 1) / QM + experts), (unsigned)((n + QN - 1) / QN));
     if (dtype == SP_BF16)
       moe_grouped_mfma_kernel<bf16_tag><<<grid, 256, 0, (hipStream_t)stream>>>(out, a, w, offsets, order, row_div, n, k,
-                                                                                experts, a_stride, out_stride);
+                                                                                experts, a_stride, out_stride, act);
     else
       moe_grouped_mfma_kernel<f16_tag><<<grid, 256, 0, (hipStream_t)stream>>>(out, a, w, offsets, order, row_div, n, k,
-                                                                               experts, a_stride, out_stride);
+                                                                               experts, a_stride, out_stride, act);
     SP_LAUNCH_CHECK();
     return SP_OK;
   }
   const dim3 grid((unsigned)((pairs + GM - 1) / GM + experts), (unsigned)((n + GN - 1) / GN));
   SP_DISPATCH_DTYPE(dtype, (moe_grouped_gemm_kernel<Tag><<<grid, 256, 0, (hipStream_t)stream>>>(
-                               out, a, w, offsets, order, row_div, pairs, n, k, experts, a_stride, out_stride)));
+                               out, a, w, offsets, order, row_div, pairs, n, k, experts, a_stride, out_stride, act)));
   SP_LAUNCH_CHECK();
   return SP_OK;
 }

@@ -12,6 +12,9 @@
 // and of sequential pre-norm models whose norm works in groups:
 //   sum + group norm      x += a  or  x += (N(a) wa + N(b) wb) / 2  (or nothing);   next = GN(x) w_next, GN = every one of
 //                         `groups` equal consecutive parts of the row divided by its own root mean square
+// and of post-norm models, whose stream is normed after every sum:
+//   scaled sum + norm     x = N(alpha x + scale * y) w, y a sublayer's result or, in the same pass, a mixture's experts
+//                         weighted and added (an expert may be the row itself) beside a gated dense branch
 // All arithmetic is fp32; h and hs are rounded once, to the projections' element type.
 #include "seq_batch.h"
 
@@ -19,13 +22,17 @@ namespace sp {
 namespace {
 
 template <typename Tag>
-__global__ void embed_scale_kernel(float* x, int64_t x_stride, const void* embed, const int64_t* ids, int width,
-                                   int64_t vocab, float scale) {
+__global__ void embed_scale_kernel(float* x, int64_t x_stride, void* lo, int64_t lo_stride, const void* embed,
+                                   const int64_t* ids, int width, int64_t vocab, float scale) {
   typedef Elem<Tag> E;
   const int64_t t = blockIdx.x;
   int64_t id = ids[t];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-  for (int i = threadIdx.x; i < width; i += blockDim.x) x[t * x_stride + i] = E::load(embed, id * width + i) * scale;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float v = E::load(embed, id * width + i) * scale;
+    x[t * x_stride + i] = v;
+    if (lo) E::store(lo, t * lo_stride + i, v);
+  }
 }
 
 // one workgroup per row: the row's own norm and, for the shift, the previous row's (recomputed: two reads of a row
@@ -461,18 +468,191 @@ add_group_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_s
   }
 }
 
+// ---- x = N(alpha x + scale * y) weight in place (+ the new x in the projections' type) -------------------------------
+// y = a, or the mixture's result assembled here: sum over k < top, in that order, of weights[t, k] times the row
+// z[place[t * top + k]] - or times x itself for an id from `experts` on - and then, with a dense branch, gate[t] * a.
+struct MixRows {
+  const void* z;               // null: no mixture
+  const int32_t* ids;
+  const int32_t* place;
+  const float* weights;
+  const float* gate;           // factor of a's row (null: 1)
+  int experts, top;
+};
+
+// rows of NV x 256 vectors of 16 bytes at most: a thread holds its part of the row in registers
+template <typename Tag, int NV>
+__global__ void __launch_bounds__(kBlock)
+post_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, MixRows mix, const float* scale, float alpha,
+                     const float* weight, void* lo, int64_t lo_stride, int width, float eps) {
+  typedef Elem<Tag> E;
+  constexpr int V = E::kVec;
+  __shared__ float red[kBlock / 64];
+  const int64_t t = blockIdx.x;
+  const int nvec = width / V;
+  float y[NV][V], xs[NV][V];
+  const float ga = (a && mix.gate) ? mix.gate[t] : 1.f;
+#pragma unroll
+  for (int u = 0; u < NV; ++u) {
+    const int vi = threadIdx.x + u * kBlock;
+    const int64_t c = (int64_t)vi * V;
+#pragma unroll
+    for (int e = 0; e < V; ++e) y[u][e] = xs[u][e] = 0.f;
+    if (vi < nvec) {
+      if (a) unpack16<Tag>(ld16((const char*)a + (t * a_stride + c) * E::kBytes), y[u]);
+#pragma unroll
+      for (int q = 0; q < V / 4; ++q) unpack16<f32_tag>(ld16(x + t * x_stride + c + 4 * q), xs[u] + 4 * q);
+    }
+  }
+  if (mix.z) {
+    float m[NV][V], self = 0.f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u)
+#pragma unroll
+      for (int e = 0; e < V; ++e) m[u][e] = 0.f;
+#pragma unroll 2
+    for (int k = 0; k < mix.top; ++k) {
+      const int64_t p = t * mix.top + k;
+      const float wk = mix.weights[p];
+      if (mix.ids[p] >= mix.experts) {                       // (the same for the whole workgroup)
+        self += wk;
+        continue;
+      }
+      const int64_t row = (int64_t)mix.place[p] * width;
+#pragma unroll
+      for (int u = 0; u < NV; ++u) {
+        const int vi = threadIdx.x + u * kBlock;
+        if (vi < nvec) {
+          float f[V];
+          unpack16<Tag>(ld16((const char*)mix.z + (row + (int64_t)vi * V) * E::kBytes), f);
+#pragma unroll
+          for (int e = 0; e < V; ++e) m[u][e] += wk * f[e];
+        }
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u)
+#pragma unroll
+      for (int e = 0; e < V; ++e) y[u][e] = m[u][e] + self * xs[u][e] + ga * y[u][e];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < NV; ++u) {
+    const int vi = threadIdx.x + u * kBlock;
+    if (vi < nvec) {
+#pragma unroll
+      for (int q = 0; q < V / 4; ++q) {
+        float s[4] = {1.f, 1.f, 1.f, 1.f};
+        if (scale) unpack16<f32_tag>(ld16(scale + (int64_t)vi * V + 4 * q), s);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float v = alpha * xs[u][4 * q + e] + s[e] * y[u][4 * q + e];
+          xs[u][4 * q + e] = v;
+          ss += v * v;
+        }
+      }
+    }
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+  for (int u = 0; u < NV; ++u) {
+    const int vi = threadIdx.x + u * kBlock;
+    if (vi < nvec) {
+      const int64_t c = (int64_t)vi * V;
+#pragma unroll
+      for (int q = 0; q < V / 4; ++q) {
+        float w[4];
+        unpack16<f32_tag>(ld16(weight + c + 4 * q), w);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) xs[u][4 * q + e] *= inv * w[e];
+        st16(x + t * x_stride + c + 4 * q, pack16<f32_tag>(xs[u] + 4 * q));
+      }
+      if (lo) st16((char*)lo + (t * lo_stride + c) * E::kBytes, pack16<Tag>(xs[u]));
+    }
+  }
+}
+
+// any width and alignment; the row's sum waits in LDS (a thread reads back only what it wrote)
+template <typename Tag>
+__global__ void __launch_bounds__(kBlock)
+post_norm_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, MixRows mix, const float* scale, float alpha,
+                 const float* weight, void* lo, int64_t lo_stride, int width, float eps) {
+  typedef Elem<Tag> E;
+  extern __shared__ float rowbuf[];
+  __shared__ float red[kBlock / 64];
+  const int64_t t = blockIdx.x;
+  const float ga = (a && mix.gate) ? mix.gate[t] : 1.f;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float xv = x[t * x_stride + i];
+    float y = a ? E::load(a, t * a_stride + i) : 0.f;
+    if (mix.z) {
+      float m = 0.f, self = 0.f;
+      for (int k = 0; k < mix.top; ++k) {
+        const int64_t p = t * mix.top + k;
+        if (mix.ids[p] >= mix.experts) self += mix.weights[p];
+        else m += mix.weights[p] * E::load(mix.z, (int64_t)mix.place[p] * width + i);
+      }
+      y = m + self * xv + ga * y;
+    }
+    const float v = alpha * xv + (scale ? scale[i] : 1.f) * y;
+    rowbuf[i] = v;
+    ss += v * v;
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float v = rowbuf[i] * (inv * weight[i]);
+    x[t * x_stride + i] = v;
+    if (lo) E::store(lo, t * lo_stride + i, v);
+  }
+}
+
 }  // namespace
 }  // namespace sp
 
 using namespace sp;
 
-extern "C" int sp_embed_scale(float* x, int64_t x_stride, const void* embed, const int64_t* ids, int64_t num_tokens,
-                              int width, int64_t vocab, float scale, int dtype, void* stream) {
+extern "C" int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a_stride, const void* z, const int32_t* ids,
+                            const int32_t* place, const float* weights, const float* gate, int experts, int top,
+                            const float* scale, float alpha, const float* weight, void* lo, int64_t lo_stride,
+                            int64_t num_tokens, int width, float eps, int dtype, void* stream) {
+  SP_CHECK_ARG(num_tokens >= 0 && width > 0 && width <= 15360);
+  if (num_tokens == 0) return SP_OK;
+  SP_CHECK_ARG(x && weight && x_stride >= width && (a || z) && (!a || a_stride >= width) && (!lo || lo_stride >= width));
+  SP_CHECK_ARG(z ? (ids && place && weights && experts > 0 && top > 0) : !gate);
+  const sp::MixRows mix{z, ids, place, weights, gate, experts, top};
+  // rows of 16-byte vectors that 256 threads hold in registers: the vector kernel; anything else: the scalar one
+  const int vecn = dtype == SP_F32 ? 4 : 8, esize = dtype == SP_F32 ? 4 : 2;
+  auto al = [&](const void* p, int64_t stride, int elem_bytes) {
+    return !p || ((((uintptr_t)p) & 15) == 0 && (stride * elem_bytes) % 16 == 0);
+  };
+  if (width % vecn == 0 && width / vecn <= 4 * kBlock && al(x, x_stride, 4) && al(a, a_stride, esize) && al(z, 0, esize) &&
+      al(lo, lo_stride, esize) && al(weight, 0, 4) && al(scale, 0, 4)) {
+    const int nv = (width / vecn + kBlock - 1) / kBlock;
+#define SP_PN(NV)                                                                                                       \
+  SP_DISPATCH_DTYPE(dtype, (post_norm_vec_kernel<Tag, NV><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(  \
+                               x, x_stride, a, a_stride, mix, scale, alpha, weight, lo, lo_stride, width, eps)))
+    if (nv <= 1) SP_PN(1);
+    else if (nv <= 2) SP_PN(2);
+    else SP_PN(4);
+#undef SP_PN
+    SP_LAUNCH_CHECK();
+    return SP_OK;
+  }
+  SP_DISPATCH_DTYPE(dtype, (post_norm_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, (size_t)width * sizeof(float),
+                                                     (hipStream_t)stream>>>(
+                               x, x_stride, a, a_stride, mix, scale, alpha, weight, lo, lo_stride, width, eps)));
+  SP_LAUNCH_CHECK();
+  return SP_OK;
+}
+
+extern "C" int sp_embed_scale(float* x, int64_t x_stride, void* lo, int64_t lo_stride, const void* embed, const int64_t* ids,
+                              int64_t num_tokens, int width, int64_t vocab, float scale, int dtype, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && width > 0 && vocab > 0);
   if (num_tokens == 0) return SP_OK;
-  SP_CHECK_ARG(x && embed && ids && x_stride >= width);
+  SP_CHECK_ARG(x && embed && ids && x_stride >= width && (!lo || lo_stride >= width));
   SP_DISPATCH_DTYPE(dtype, (embed_scale_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(
-                               x, x_stride, embed, ids, width, vocab, scale)));
+                               x, x_stride, lo, lo_stride, embed, ids, width, vocab, scale)));
   SP_LAUNCH_CHECK();
   return SP_OK;
 }

@@ -17,7 +17,8 @@
 // is seen by every query, is not scaled and has no value.
 //
 // Further forms of the same layer (each a parameter): q and k divided per head by their root mean square after the
-// rotation; q times a number per head and times 1 + coef ln(floor((position + 1) / every) + 1); values blended with the
+// rotation, or before it and then times a learned weight per coordinate (shared by the heads); values that are the keys as
+// projected, before norm and rotation; q times a number per head and times 1 + coef ln(floor((position + 1) / every) + 1); values blended with the
 // values an earlier layer cached for the same token, v <- (1 - lambda) v + lambda v_first; scores capped as
 // cap tanh(score / cap); and, instead of the softmax, every visible key weighted by sigmoid(score + bias[head]) without
 // normalisation.  The result can be multiplied element by element with sigmoid(gate) on its way out.
@@ -90,8 +91,9 @@ qkv_rotary_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stri
 }
 
 // The same store with a wave per head: q and k can be divided by their root mean square over the head AFTER the rotation
-// (qk_norm), q scaled per head and by position, v blended with the row another layer's pool holds for the same slot.
-// A lane holds the coordinates lane, lane + 64, ... of its head (dim, vdim <= 64 * kStorePerLane).
+// (qk_norm 1) or BEFORE it, times a weight per coordinate (qk_norm 2), q scaled per head and by position, v blended with the
+// row another layer's pool holds for the same slot.  v null: the values are the keys as projected (bias included, neither
+// normed nor rotated), written by the wave that makes the key.  A lane holds the coordinates lane, lane + 64, ... of its head (dim, vdim <= 64 * kStorePerLane).
 constexpr int kStorePerLane = 4;
 template <typename Tag>
 __device__ __forceinline__ void rotated_head(float* val, const void* src, int64_t at, const float* bias, int col0, int D,
@@ -127,13 +129,49 @@ __device__ __forceinline__ void rotated_head(float* val, const void* src, int64_
   }
 }
 
+// the head before the rotation divided by its root mean square and times weight[i], then rotated; raw: the head as projected
+template <typename Tag>
+__device__ __forceinline__ void normed_rotated_head(float* val, float* raw, const void* src, int64_t at, const float* bias,
+                                                    int col0, int D, int dims, int adjacent, float pos, const float* freq,
+                                                    float mag, const float* weight, float eps, int lane) {
+  typedef Elem<Tag> E;
+  const int half = dims / 2;
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < kStorePerLane; ++u) {
+    const int i = lane + 64 * u;
+    raw[u] = i < D ? E::load(src, at + i) + (bias ? bias[col0 + i] : 0.f) : 0.f;
+    ss += raw[u] * raw[u];
+  }
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)D + eps);
+#pragma unroll
+  for (int u = 0; u < kStorePerLane; ++u) {
+    const int i = lane + 64 * u;
+    float out = 0.f;
+    if (i < D) {
+      const float x = raw[u] * inv * (weight ? weight[i] : 1.f);
+      out = x;
+      if (i < dims) {
+        const bool first = adjacent ? (i & 1) == 0 : i < half;
+        const int pi = adjacent ? (first ? i + 1 : i - 1) : (first ? i + half : i - half);
+        const int fi = adjacent ? i >> 1 : (first ? i : i - half);
+        const float y = (E::load(src, at + pi) + (bias ? bias[col0 + pi] : 0.f)) * inv * (weight ? weight[pi] : 1.f);
+        const float ang = pos * freq[fi];
+        const float c = cosf(ang) * mag, sn = sinf(ang) * mag;
+        out = first ? x * c - y * sn : x * c + y * sn;
+      }
+    }
+    val[u] = out;
+  }
+}
+
 template <typename Tag>
 __global__ void __launch_bounds__(kBlock)
 qkv_norm_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v, int64_t v_stride,
                       void* kpool, int64_t kp_stride, void* vpool, int64_t vp_stride, const int64_t* positions,
                       const int64_t* loc, const float* freq, float mag, const float* qb, const float* kb, const float* vb,
                       int H, int G, int D, int Dv, int dims, int adjacent, int norm_v, float eps, int qk_norm,
-                      const float* q_head_scale, float q_temp_coef, int q_temp_every, const void* v_first,
+                      const float* q_norm_w, const float* k_norm_w, const float* q_head_scale, float q_temp_coef, int q_temp_every, const void* v_first,
                       int64_t vf_stride, const float* v_mix) {
   typedef Elem<Tag> E;
   const int64_t t = blockIdx.x;
@@ -143,16 +181,35 @@ qkv_norm_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stride
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
   float qmul = 1.f;
   if (q_temp_every > 0) qmul = 1.f + q_temp_coef * logf((float)((ipos + 1) / q_temp_every) + 1.f);
-  for (int job = wave; job < H + 2 * G; job += waves) {
-    float val[kStorePerLane];
+  for (int job = wave; job < H + (v ? 2 * G : G); job += waves) {
+    float val[kStorePerLane], raw[kStorePerLane];
     if (job < H + G) {
       const bool isq = job < H;
       const int h = isq ? job : job - H;
       const void* src = isq ? q : k;
       const int64_t at = t * (isq ? q_stride : k_stride) + (int64_t)h * D;
-      rotated_head<Tag>(val, src, at, isq ? qb : kb, h * D, D, dims, adjacent, pos, freq, mag, lane);
+      if (qk_norm == 2) {
+        normed_rotated_head<Tag>(val, raw, src, at, isq ? qb : kb, h * D, D, dims, adjacent, pos, freq, mag,
+                                 isq ? q_norm_w : k_norm_w, eps, lane);
+        if (!isq && !v) {
+#pragma unroll
+          for (int u = 0; u < kStorePerLane; ++u) {
+            const int i = lane + 64 * u;
+            if (i < D) E::store(vpool, slot * vp_stride + (int64_t)h * D + i, raw[u]);
+          }
+        }
+      } else {
+        rotated_head<Tag>(val, src, at, isq ? qb : kb, h * D, D, dims, adjacent, pos, freq, mag, lane);
+        if (!isq && !v) {
+#pragma unroll
+          for (int u = 0; u < kStorePerLane; ++u) {
+            const int i = lane + 64 * u;
+            if (i < D) E::store(vpool, slot * vp_stride + (int64_t)h * D + i, E::load(k, at + i) + (kb ? kb[h * D + i] : 0.f));
+          }
+        }
+      }
       float mul = 1.f;
-      if (qk_norm) {
+      if (qk_norm == 1) {
         float ss = 0.f;
 #pragma unroll
         for (int u = 0; u < kStorePerLane; ++u) ss += val[u] * val[u];       // (coordinates past D are zeros)
@@ -599,22 +656,25 @@ extern "C" int sp_qkv_rotary_store(void* q, int64_t q_stride, const void* k, int
                                    const int64_t* positions, const int64_t* loc, const float* freq, float mag,
                                    const float* q_bias, const float* k_bias, const float* v_bias, int64_t num_tokens,
                                    int heads, int kv_heads, int dim, int vdim, int rot_dims, int adjacent, int norm_values,
-                                   float eps, int qk_norm, const float* q_head_scale, float q_temp_coef, int q_temp_every,
-                                   const void* v_first, int64_t vf_stride, const float* v_mix, int dtype, void* stream) {
+                                   float eps, int qk_norm, const float* q_norm_weight, const float* k_norm_weight,
+                                   const float* q_head_scale, float q_temp_coef, int q_temp_every, const void* v_first,
+                                   int64_t vf_stride, const float* v_mix, int dtype, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0);
   SP_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim);
+  SP_CHECK_ARG(qk_norm >= 0 && qk_norm <= 2 && (qk_norm == 2 || (!q_norm_weight && !k_norm_weight)));
   if (num_tokens == 0) return SP_OK;
-  SP_CHECK_ARG(q && k && v && kpool && vpool && positions && loc && (freq || rot_dims == 0));
-  SP_CHECK_ARG(q_stride >= (int64_t)heads * dim && k_stride >= (int64_t)kv_heads * dim && v_stride >= (int64_t)kv_heads * vdim);
+  SP_CHECK_ARG(q && k && kpool && vpool && positions && loc && (freq || rot_dims == 0));
+  SP_CHECK_ARG(q_stride >= (int64_t)heads * dim && k_stride >= (int64_t)kv_heads * dim);
+  SP_CHECK_ARG(v ? v_stride >= (int64_t)kv_heads * vdim : (dim == vdim && !v_bias && !norm_values && !v_first));
   SP_CHECK_ARG(kp_stride >= (int64_t)kv_heads * dim && vp_stride >= (int64_t)kv_heads * vdim);
   SP_CHECK_ARG(q_temp_every >= 0 && (!v_first || (v_mix && vf_stride >= (int64_t)kv_heads * vdim)));
-  if (qk_norm || q_head_scale || q_temp_every > 0 || v_first) {      // the wave-per-head form
+  if (qk_norm || q_head_scale || q_temp_every > 0 || v_first || !v) {      // the wave-per-head form
     if (dim > 64 * kStorePerLane || vdim > 64 * kStorePerLane) return SP_ERR_UNSUPPORTED;
     SP_DISPATCH_DTYPE(dtype, (qkv_norm_store_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(
                                  q, q_stride, k, k_stride, v, v_stride, kpool, kp_stride, vpool, vp_stride, positions, loc,
                                  freq, mag, q_bias, k_bias, v_bias, heads, kv_heads, dim, vdim, rot_dims, adjacent,
-                                 norm_values, eps, qk_norm, q_head_scale, q_temp_coef, q_temp_every, v_first, vf_stride,
-                                 v_mix)));
+                                 norm_values, eps, qk_norm, q_norm_weight, k_norm_weight, q_head_scale, q_temp_coef,
+                                 q_temp_every, v_first, vf_stride, v_mix)));
     SP_LAUNCH_CHECK();
     return SP_OK;
   }

@@ -429,6 +429,30 @@ class ReluSquareFF(nn.Module):
         self.act = ReluSquare()
 
     def forward(self, h: torch.Tensor):
+        if not self.extra_rows:
+            return _native.linear(_native.linear_relu_square(h, self.up), self.down)
         a = _native.linear(h, self.up)
-        y = _native.linear(self.act(a[:, :self.ff]), self.down)
-        return (y, a[:, self.ff:]) if self.extra_rows else y
+        return _native.linear(self.act(a[:, :self.ff]), self.down), a[:, self.ff:]
+
+
+class PostNorm(nn.Module):
+    """How a sublayer's result y joins an fp32 residual stream that is normed AFTER the sum:
+    x <- N(alpha x + scale * y) * weight, N = division by the row's root mean square, scale a learned vector (``layer_scale``)
+    or 1.  The stream itself is what the next sublayer reads, so the call returns it in the projections' dtype.  y is a
+    tensor, or moe.MixtureRows - a mixture whose weighted sum (and identity experts, and gated dense branch) is formed in the
+    same pass over the row."""
+
+    def __init__(self, width: int, eps: float = 1e-6, alpha: float = 1.0, layer_scale: bool = False) -> None:
+        super().__init__()
+        f32 = dict(dtype=torch.float32)
+        self.weight = nn.Parameter(torch.ones(width, **f32), requires_grad=False)
+        self.scale = nn.Parameter(torch.ones(width, **f32), requires_grad=False) if layer_scale else None
+        self.variance_epsilon, self.alpha = eps, alpha
+
+    def forward(self, x: torch.Tensor, y, dtype: torch.dtype, want_lo: bool = True) -> Optional[torch.Tensor]:
+        mix = {}
+        if not isinstance(y, torch.Tensor):
+            mix = dict(z=y.z, ids=y.ids, place=y.place, weights=y.weights, gate=y.gate, experts=y.experts)
+            y = y.dense
+        return _native.post_norm(x, y, self.weight.data, self.variance_epsilon, self.alpha, dtype,
+                                 scale=None if self.scale is None else self.scale.data, want_lo=want_lo, **mix)

@@ -45,6 +45,11 @@ def _kikurax_config(raw: dict, context_len=None, tensor_shapes=None, **_kw):
     return KikuraxConfig(raw, context_len=context_len or 8192, tensor_shapes=tensor_shapes)
 
 
+def _monolix_config(raw: dict, context_len=None, **_kw):
+    from .monolix import MonolixConfig
+    return MonolixConfig(raw, context_len=context_len or 8192)
+
+
 def _llama_class():
     from .llama import LlamaForCausalLM
     return LlamaForCausalLM
@@ -75,6 +80,11 @@ def _kikurax_class():
     return KikuraxForCausalLM
 
 
+def _monolix_class():
+    from .monolix import MonolixForCausalLM
+    return MonolixForCausalLM
+
+
 # architecture name -> (configuration from config.json's dict, model class); both lazy so that naming a model does not
 # import the others
 MODELS = {
@@ -83,6 +93,7 @@ MODELS = {
     "Sominex": (_sominex_config, _sominex_class),
     "Toredra": (_toredra_config, _toredra_class),
     "Kikurax": (_kikurax_config, _kikurax_class),
+    "Monolix": (_monolix_config, _monolix_class),
 }
 
 
