@@ -1,7 +1,7 @@
-"""bench.py --mode hybrid / --mode sominex / --mode toredra / --mode kikurax: prefill and decode throughput of the Tizalorn /
-the Sominex / the Toredra / the Kikurax design at layer sizes of real models (random weights), beside a Llama of the same
-width and depth on the same engine path (the Toredra mode also runs Sominex, the Kikurax mode Sominex and Toredra: their
-nearest relatives), and a per-kernel table: every HIP kernel
+"""bench.py --mode hybrid / --mode sominex / --mode toredra / --mode kikurax / --mode monolix: prefill and decode throughput of
+the Tizalorn / the Sominex / the Toredra / the Kikurax / the Monolix design at layer sizes of real models (random weights),
+beside a Llama of the same width and depth on the same engine path (the Toredra mode also runs Sominex, the Kikurax mode
+Sominex and Toredra, the Monolix mode Kikurax: their nearest relatives), and a per-kernel table: every HIP kernel
 (and library product) of both models timed inside an eager prefill batch and an eager decode step, with the time its
 algorithmic bytes and flops would take at the chip's peaks (fraction of roofline).
 
@@ -93,6 +93,20 @@ def kikurax_config(width: int, layers: int, context_len: int):
     raw = {"architecture": "Kikurax", "vocab": 128256, "width": width, "norm": {"eps": 1e-5, "groups": 4},
            "embedding": {"scale": float(width) ** 0.5}, "layers": [{**pattern[i % 4], "mlp": moe} for i in range(layers)]}
     return KikuraxConfig(raw, context_len=context_len, low_rank=64)
+
+
+def monolix_config(width: int, layers: int, context_len: int):
+    """attention heads of 128 with a quarter as many key/value heads and rotation on half of each head; 32 experts and 8
+    identity experts in 4 groups of which 2 are kept, 4 chosen, and a shared expert of the model's width"""
+    from scratchpad_amd.monolix import MonolixConfig
+    att = {"type": "attention",
+           "mixer": {"heads": width // 128, "kv_heads": max(1, width // 512), "dim": 128, "vdim": 128, "scale": 0.09,
+                     "rot": {"base": 500000.0, "dims": 64}}}
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "shared": {"ff": width},
+           "router": {"experts": 32, "top": 4, "identity": 8, "groups": {"count": 4, "keep": 2}}}
+    raw = {"architecture": "Monolix", "vocab": 128256, "width": width, "norm": {"eps": 1e-5}, "postln_alpha": 2.5,
+           "layers": [{**att, "mlp": moe} for _ in range(layers)]}
+    return MonolixConfig(raw, context_len=context_len)
 
 
 def llama_config(width: int, layers: int, context_len: int):
@@ -235,6 +249,12 @@ def instrument(clock: KernelClock, cfg):
         p, w = a[0], a[1]
         return _nbytes(p, w, out), 2 * p.shape[0] * w.shape[0] * w.shape[1], VECTOR32
 
+    def join(a, k, out):         # the stream in and out, the result or a mixture's rows (identity experts' have none), the copy
+        rows = 0
+        if k.get("z") is not None:
+            rows = int((k["ids"] < k["experts"]).sum()) * k["z"].shape[1] * k["z"].element_size()
+        return 2 * _nbytes(a[0]) + _nbytes(a[1], a[2], out) + rows, 0, MATRIX
+
     costs = {"embed_bigram_norm": io, "add_scalar_norm": io, "scalar_norm": io, "polynorm": io, "gate_heads": io,
              "token_shift": io, "wkv_decay": io, "wkv_recurrence": wkv, "rotary_interleaved": io, "latent_kv_store": io,
              "latent_attention": latent, "moe_route": io, "moe_align": io, "moe_grouped_gemm": grouped, "moe_glu": io,
@@ -244,7 +264,7 @@ def instrument(clock: KernelClock, cfg):
              "window_attention": window, "small_linear_f32": small, "causal_conv_silu": io, "mamba2_scan": scan,
              "gated_group_norm": io, "mlstm_scan": mlstm, "moe_route_softmax": io,
              "gated_add_norm": io, "relu_square": io, "scale_softcap": io, "delta_gates": io, "delta_recurrence": delta,
-             "hgrn2_scan": hgrn, "add_group_norm": io, "lowrank_gate": lowrank, "gated_delta_scan": gdelta}
+             "hgrn2_scan": hgrn, "linear_relu_square": gemm, "post_norm": join, "add_group_norm": io, "lowrank_gate": lowrank, "gated_delta_scan": gdelta}
     for name, cost in costs.items():
         saved[name] = getattr(N, name)
         setattr(N, name, clock.record(name, saved[name], cost))
@@ -373,7 +393,7 @@ def hybrid_main(args, design: str = "tizalorn"):
     runs = []
     for w in widths:
         row = {"width": w, "layers": layers}
-        beside = {"toredra": ("sominex", "llama"), "kikurax": ("sominex", "toredra", "llama")}.get(design, ("llama",))
+        beside = {"toredra": ("sominex", "llama"), "kikurax": ("sominex", "toredra", "llama"), "monolix": ("kikurax", "llama")}.get(design, ("llama",))
         for model in (design, *beside):
             cmd = [sys.executable, "-u", os.path.abspath(__file__), "--child", model, "--width", str(w), "--layers", str(layers),
                    "--bs", str(args.bs), "--ctx", str(args.ctx), "--steps", str(args.steps), "--warmup", str(args.warmup),
@@ -406,7 +426,7 @@ def child_main():
     import sys
     sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
     ap = argparse.ArgumentParser()
-    ap.add_argument("--child", required=True, choices=["tizalorn", "sominex", "toredra", "kikurax", "llama"])
+    ap.add_argument("--child", required=True, choices=["tizalorn", "sominex", "toredra", "kikurax", "monolix", "llama"])
     for name in ("width", "layers", "bs", "ctx", "steps", "warmup", "max-prefill-tokens"):
         ap.add_argument("--" + name, type=int, required=True)
     ap.add_argument("--no-graph", action="store_true")
@@ -416,7 +436,7 @@ def child_main():
         raise SystemExit(DISABLED)
     torch.cuda.set_device(0)
     ctx_len = a.ctx + 2 * (a.steps + a.warmup) + 16
-    cfg = {"sominex": sominex_config, "toredra": toredra_config, "kikurax": kikurax_config, "llama": llama_config}[a.child](a.width, a.layers, ctx_len)
+    cfg = {"sominex": sominex_config, "toredra": toredra_config, "kikurax": kikurax_config, "monolix": monolix_config, "llama": llama_config}[a.child](a.width, a.layers, ctx_len)
     out = run_model(cfg, a, not a.no_kernel_table)
     print("RESULT " + json.dumps(out), flush=True)
 

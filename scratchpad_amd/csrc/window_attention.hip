@@ -94,10 +94,11 @@ qkv_rotary_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stri
 // (qk_norm 1) or BEFORE it, times a weight per coordinate (qk_norm 2), q scaled per head and by position, v blended with the
 // row another layer's pool holds for the same slot.  v null: the values are the keys as projected (bias included, neither
 // normed nor rotated), written by the wave that makes the key.  A lane holds the coordinates lane, lane + 64, ... of its head (dim, vdim <= 64 * kStorePerLane).
+// The token's angles are the same for all its heads: their cosines and sines (times mag) wait in LDS.
 constexpr int kStorePerLane = 4;
 template <typename Tag>
 __device__ __forceinline__ void rotated_head(float* val, const void* src, int64_t at, const float* bias, int col0, int D,
-                                             int dims, int adjacent, float pos, const float* freq, float mag, int lane) {
+                                             int dims, int adjacent, const float* cosine, const float* sine, int lane) {
   typedef Elem<Tag> E;
   const int half = dims / 2;
 #pragma unroll
@@ -120,8 +121,7 @@ __device__ __forceinline__ void rotated_head(float* val, const void* src, int64_
           fi = first ? i : i - half;
         }
         const float y = E::load(src, at + pi) + (bias ? bias[col0 + pi] : 0.f);
-        const float ang = pos * freq[fi];
-        const float c = cosf(ang) * mag, sn = sinf(ang) * mag;
+        const float c = cosine[fi], sn = sine[fi];
         out = first ? x * c - y * sn : x * c + y * sn;
       }
     }
@@ -132,8 +132,8 @@ __device__ __forceinline__ void rotated_head(float* val, const void* src, int64_
 // the head before the rotation divided by its root mean square and times weight[i], then rotated; raw: the head as projected
 template <typename Tag>
 __device__ __forceinline__ void normed_rotated_head(float* val, float* raw, const void* src, int64_t at, const float* bias,
-                                                    int col0, int D, int dims, int adjacent, float pos, const float* freq,
-                                                    float mag, const float* weight, float eps, int lane) {
+                                                    int col0, int D, int dims, int adjacent, const float* cosine,
+                                                    const float* sine, const float* weight, float eps, int lane) {
   typedef Elem<Tag> E;
   const int half = dims / 2;
   float ss = 0.f;
@@ -156,8 +156,7 @@ __device__ __forceinline__ void normed_rotated_head(float* val, float* raw, cons
         const int pi = adjacent ? (first ? i + 1 : i - 1) : (first ? i + half : i - half);
         const int fi = adjacent ? i >> 1 : (first ? i : i - half);
         const float y = (E::load(src, at + pi) + (bias ? bias[col0 + pi] : 0.f)) * inv * (weight ? weight[pi] : 1.f);
-        const float ang = pos * freq[fi];
-        const float c = cosf(ang) * mag, sn = sinf(ang) * mag;
+        const float c = cosine[fi], sn = sine[fi];
         out = first ? x * c - y * sn : x * c + y * sn;
       }
     }
@@ -166,7 +165,7 @@ __device__ __forceinline__ void normed_rotated_head(float* val, float* raw, cons
 }
 
 template <typename Tag>
-__global__ void __launch_bounds__(kBlock)
+__global__ void __launch_bounds__(1024)
 qkv_norm_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v, int64_t v_stride,
                       void* kpool, int64_t kp_stride, void* vpool, int64_t vp_stride, const int64_t* positions,
                       const int64_t* loc, const float* freq, float mag, const float* qb, const float* kb, const float* vb,
@@ -178,6 +177,13 @@ qkv_norm_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stride
   const int64_t ipos = positions[t];
   const float pos = (float)ipos;
   const int64_t slot = loc[t];
+  __shared__ float cosine[32 * kStorePerLane], sine[32 * kStorePerLane];      // dims <= D <= 64 * kStorePerLane
+  for (int i = threadIdx.x; i < dims / 2; i += blockDim.x) {
+    const float ang = pos * freq[i];
+    cosine[i] = cosf(ang) * mag;
+    sine[i] = sinf(ang) * mag;
+  }
+  __syncthreads();
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
   float qmul = 1.f;
   if (q_temp_every > 0) qmul = 1.f + q_temp_coef * logf((float)((ipos + 1) / q_temp_every) + 1.f);
@@ -189,7 +195,7 @@ qkv_norm_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stride
       const void* src = isq ? q : k;
       const int64_t at = t * (isq ? q_stride : k_stride) + (int64_t)h * D;
       if (qk_norm == 2) {
-        normed_rotated_head<Tag>(val, raw, src, at, isq ? qb : kb, h * D, D, dims, adjacent, pos, freq, mag,
+        normed_rotated_head<Tag>(val, raw, src, at, isq ? qb : kb, h * D, D, dims, adjacent, cosine, sine,
                                  isq ? q_norm_w : k_norm_w, eps, lane);
         if (!isq && !v) {
 #pragma unroll
@@ -199,7 +205,7 @@ qkv_norm_store_kernel(void* q, int64_t q_stride, const void* k, int64_t k_stride
           }
         }
       } else {
-        rotated_head<Tag>(val, src, at, isq ? qb : kb, h * D, D, dims, adjacent, pos, freq, mag, lane);
+        rotated_head<Tag>(val, src, at, isq ? qb : kb, h * D, D, dims, adjacent, cosine, sine, lane);
         if (!isq && !v) {
 #pragma unroll
           for (int u = 0; u < kStorePerLane; ++u) {
@@ -670,7 +676,10 @@ extern "C" int sp_qkv_rotary_store(void* q, int64_t q_stride, const void* k, int
   SP_CHECK_ARG(q_temp_every >= 0 && (!v_first || (v_mix && vf_stride >= (int64_t)kv_heads * vdim)));
   if (qk_norm || q_head_scale || q_temp_every > 0 || v_first || !v) {      // the wave-per-head form
     if (dim > 64 * kStorePerLane || vdim > 64 * kStorePerLane) return SP_ERR_UNSUPPORTED;
-    SP_DISPATCH_DTYPE(dtype, (qkv_norm_store_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(
+    // four waves take a prompt token's heads in turn; the few tokens of a decode step get a wave per head (16 at most)
+    const int jobs = heads + (v ? 2 : 1) * kv_heads;
+    const int threads = num_tokens > 256 ? kBlock : 64 * (jobs < 4 ? 4 : (jobs > 16 ? 16 : jobs));
+    SP_DISPATCH_DTYPE(dtype, (qkv_norm_store_kernel<Tag><<<dim3((unsigned)num_tokens), threads, 0, (hipStream_t)stream>>>(
                                  q, q_stride, k, k_stride, v, v_stride, kpool, kp_stride, vpool, vp_stride, positions, loc,
                                  freq, mag, q_bias, k_bias, v_bias, heads, kv_heads, dim, vdim, rot_dims, adjacent,
                                  norm_values, eps, qk_norm, q_norm_weight, k_norm_weight, q_head_scale, q_temp_coef,
