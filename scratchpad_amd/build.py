@@ -14,8 +14,10 @@ CSRC = os.path.join(PKG, "csrc")
 LIB = os.path.join(PKG, "lib", "libscratchpad_hip.so")
 OBJ = os.path.join(ROOT, "build", "obj")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
+# scalar fp32 instructions only (no packed-fp32 forms): some of those have given wrong results on this hardware now and then
+_NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unknown-warning-option"]
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-fvisibility=hidden",
-         "-Wno-unused-value"]
+         "-Wno-unused-value"] + _NO_PACKED_F32
 # elementwise.hip reproduces torch's per-op rounding (round16(a*b) - round16(c*d)); the default
 # -ffp-contract=fast lets the backend fuse that into v_fma_f16 whatever the source pragmas say
 # extend_mfma.hip: without -fno-honor-nans every fmaxf on an MFMA result is preceded by a canonicalising
@@ -29,11 +31,6 @@ PER_FILE_FLAGS = {"elementwise.hip": ["-ffp-contract=off"], "allreduce.hip": ["-
                   # accumulation registers belong to its assembly text alone: compile_w64 below / tools/w64_asm.py.  The
                   # atomic optimizer would turn the persistent form's ticket draw into atomic + full wait + broadcast.
                   "extend_w64.hip": ["-fno-honor-nans", "-fno-slp-vectorize", "-std=c++20", "-mllvm", "-amdgpu-atomic-optimizer-strategy=None"]}
-# fp32 state and residual kernels: scalar fp32 instructions only (no packed-fp32 forms)
-_NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unknown-warning-option"]
-for _f in ("scalar_norm.hip", "wkv.hip", "latent_attention.hip", "moe.hip", "stream_norm.hip", "window_attention.hip",
-           "ssm.hip", "mlstm.hip", "delta_rule.hip", "hgrn.hip", "gated_delta.hip"):
-    PER_FILE_FLAGS[_f] = list(_NO_PACKED_F32)
 # Sources a model family needs beyond these: a model class names them (NATIVE_SOURCES) and build_native(only=...) makes
 # a library of just those, so the first start of a small model does not compile the attention kernels of another.
 CORE_SOURCES = ["elementwise.hip", "gemm_skinny.hip", "sampling.hip"]

@@ -11,7 +11,7 @@ for f in scratchpad_amd/csrc/*.hip; do
     elementwise.hip) extra="-ffp-contract=off";;
     extend_mfma.hip) extra="-fno-honor-nans";;
   esac
-  /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -fvisibility=hidden -Wno-unused-value \
+  /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -fvisibility=hidden -Wno-unused-value -Xclang -target-feature -Xclang -packed-fp32-ops -Wno-unknown-warning-option \
     ${SP_STAMP_DEFS:--DSP_EXTEND_STAMPS} $extra -c $f -o build/stamps/$(basename $f .hip).o &
 done
 wait

@@ -6,7 +6,7 @@ set -e
 cd "$(dirname "$0")/.."
 NAME=$1; shift
 mkdir -p build/variants
-/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -fvisibility=hidden -Wno-unused-value -fno-honor-nans \
+/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -fvisibility=hidden -Wno-unused-value -Xclang -target-feature -Xclang -packed-fp32-ops -Wno-unknown-warning-option -fno-honor-nans \
   -DSP_EXTEND_ONLY_HEADLINE "$@" -c scratchpad_amd/csrc/extend_mfma.hip -o build/variants/extend_mfma_$NAME.o
 OBJS=$(ls build/obj/*.o | grep -v extend_mfma.o)
 /opt/rocm/bin/hipcc --offload-arch=gfx950 -shared -fPIC -o scratchpad_amd/lib/libscratchpad_hip_$NAME.so $OBJS build/variants/extend_mfma_$NAME.o
