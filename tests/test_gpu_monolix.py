@@ -82,7 +82,7 @@ def test_post_norm_kernel_in_every_form(W, alpha):
                     assert out is None
 
 
-@pytest.mark.parametrize("E,top,count,keep", [(12, 3, 2, 1), (12, 4, 6, 2), (5, 5, 1, 1), (70, 1, 1, 1), (130, 6, 65, 4),
+@pytest.mark.parametrize("E,top,count,keep", [(14, 3, 2, 1), (12, 4, 6, 2), (5, 5, 1, 1), (70, 1, 1, 1), (130, 6, 65, 4),
                                               (9, 3, 9, 3), (8, 2, 4, 4)])
 def test_router_choice_in_groups_with_corrections_of_either_sign(E, top, count, keep):
     from scratchpad_amd import _native
