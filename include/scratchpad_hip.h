@@ -31,7 +31,7 @@
 extern "C" {
 #endif
 
-#define SP_ABI_VERSION 14
+#define SP_ABI_VERSION 15
 #define SP_API __attribute__((visibility("default")))
 
 typedef enum { SP_F32 = 0, SP_F16 = 1, SP_BF16 = 2, SP_FP8_E5M2 = 3 /* KV pool only */ } sp_dtype;
@@ -338,7 +338,8 @@ SP_API int sp_top_k_top_p_min_p_renorm(const float* probs, int64_t row_stride, c
  *      `epilogue` (ABI 6): 0 = out[M, N] as above.  1 = w is the merged gate|up matrix [2 N, K] of LlamaMLP
  *      (gate rows first; MergedColumnParallelLinear, linear.py:423-470) and out[M, N] = SiluAndMul of the projection
  *      (nn/layers/activation.py:21-31), bit for bit the plain call followed by sp_silu_and_mul: gate_up_proj +
- *      act_fn (nn/models/llama/llama.py:62-66) in one launch.  2 (ABI 14) = max(out, 0)^2.          */
+ *      act_fn (nn/models/llama/llama.py:62-66) in one launch.  2 (ABI 14) = max(out, 0)^2.
+ *      3 (ABI 15) = as 1 with gelu_tanh(gate) * up: bit for bit the plain call followed by sp_gelu_tanh_and_mul. */
 SP_API int sp_gemm_skinny(void* out, const void* x, const void* w, int M, int N, int K, int64_t x_stride,
                    int64_t w_stride, int64_t out_stride, int epilogue, int dtype, void* stream);
 
@@ -450,17 +451,29 @@ SP_API int sp_wkv_recurrence(void* out, const void* r, const void* k, const void
 SP_API int sp_rotary_interleaved(void* x, const int64_t* positions, const float* freq, float mag, int64_t num_tokens,
                                  int heads, int rot_dim, int64_t token_stride, int64_t head_stride, int offset, int dtype,
                                  void* stream);
-/* pool[loc[t]] = [ dkv[t, :rank] / rms * norm_w | dkv[t, rank : rank + rot_dim] with its first rot_dims rotated ] */
+/* pool[loc[t]] = [ dkv[t, :rank] / rms * norm_w | dkv[t, rank : rank + rot_dim] with its first rot_dims rotated ]
+ * (ABI 15) q (optional): q[t, h, q_offset .. q_offset + rot_dims) rotated in place for every head in the same launch; pool
+ * null: nothing is stored (a layer that attends to another layer's rows).                                              */
 SP_API int sp_latent_kv_store(void* pool, int64_t pool_stride, const void* dkv, int64_t dkv_stride, const float* norm_w,
+                              void* q, int64_t q_stride, int64_t q_head_stride, int q_offset, int heads,
                               const int64_t* positions, const float* freq, float mag, const int64_t* loc,
                               int64_t num_tokens, int rank, int rot_dim, int rot_dims, float eps, int dtype, void* stream);
 /* Causal multi-query attention over pool rows [rank | rot_dim]: score = (q_lat . row[:rank] + q_rot . row[rank:]) * scale,
- * softmax in fp32, out = sum p * row[:rank].  q_lat, out: [heads, T, rank]; q_rot: x[t * token_stride + h * head_stride + ..].
- * A token at position p of its request sees the request's positions 0 .. p through req_to_token.  rank <= 1024.  */
-SP_API int sp_latent_attention(void* out, const void* q_lat, const void* q_rot, const void* pool, int64_t pool_stride,
-                               const int32_t* req_to_token, int64_t table_stride, int64_t num_tokens, int heads, int rank,
-                               int rot_dim, int64_t qrot_token_stride, int64_t qrot_head_stride, float scale,
-                               SP_SEQ_PARAMS, int dtype, void* stream);
+ * softmax in fp32, out = sum p * row[:rank].  q_lat, out: x[t * lat_token_stride + h * lat_head_stride + ..]; q_rot likewise.
+ * A token at position p of its request sees the request's positions 0 .. p through req_to_token.  rank <= 1024.
+ * (ABI 15) matrix != 0: 16-bit types with rank and rot_dim multiples of 8, rank <= 512, rank + rot_dim <= 576 and 16-byte
+ * aligned rows run on the matrix cores; splits > 1 then shares the keys of every query over that many workgroups, which join
+ * through the workspace (fp32, splits * T * heads * (rank + 2) values).                                              */
+SP_API int sp_latent_attention(void* out, const void* q_lat, int64_t lat_token_stride, int64_t lat_head_stride,
+                               const void* q_rot, const void* pool, int64_t pool_stride, const int32_t* req_to_token,
+                               int64_t table_stride, int64_t num_tokens, int heads, int rank, int rot_dim,
+                               int64_t qrot_token_stride, int64_t qrot_head_stride, float scale, int matrix, int splits,
+                               float* workspace, int64_t workspace_floats, SP_SEQ_PARAMS, int dtype, void* stream);
+/* (ABI 15) A product per head: out[t, h, j] = sum_i w[h, j, i] x[t, h, i], w [heads, n, k] contiguous, x and out with a token
+ * and a head stride; with gate ([T, heads * n], row stride gate_stride) the result is multiplied with sigmoid(gate).   */
+SP_API int sp_head_linear(void* out, int64_t out_stride, int64_t out_head_stride, const void* x, int64_t x_stride,
+                          int64_t x_head_stride, const void* w, const void* gate, int64_t gate_stride, int64_t num_tokens,
+                          int heads, int n, int k, int dtype, void* stream);
 
 /* Router: z = router x in fp32, s = sigmoid(z), choice = s + correction; with groups > 1 only experts of the `keep`
  * groups with the largest (sum of the group's two largest choices) can win; ids [T, top] = the largest choices,
@@ -495,9 +508,11 @@ SP_API int sp_moe_softmax_topk(int32_t* ids, float* weights, float* gate, const 
                                float scale, int renorm, void* stream);
 
 /* ---- fp32 residual stream of parallel-sublayer layers (csrc/stream_norm.hip) ------------------------------------- */
-/* x[t] = embed[ids[t]] * scale  (x fp32, embed in `dtype`); lo (optional, ABI 14): the same row in `dtype` */
+/* x[t] = embed[ids[t]] * scale  (x fp32, embed in `dtype`); lo (optional, ABI 14): the same row in `dtype`.
+ * (ABI 15) table (optional, in `dtype`, [table_rows, width]): x[t] += table[positions[t]], the sum in fp32           */
 SP_API int sp_embed_scale(float* x, int64_t x_stride, void* lo, int64_t lo_stride, const void* embed, const int64_t* ids,
-                          int64_t num_tokens, int width, int64_t vocab, float scale, int dtype, void* stream);
+                          const void* table, const int64_t* positions, int64_t table_rows, int64_t num_tokens, int width,
+                          int64_t vocab, float scale, int dtype, void* stream);
 /* h[t] = x[t] / sqrt(mean(x[t]^2) + eps) * weight -> out_h; hs[t] = h[t] + (h[t-1] - h[t]) * mu -> out_hs (both in
  * `dtype`, either may be null; out_hs null: a plain weighted norm, the request description is not read).  The row before
  * a step's first row is state[request slot] (zeros at a sequence's first token).                                    */
@@ -547,9 +562,10 @@ SP_API int sp_pool_blocks(void* kpooled, void* vpooled, const void* kpool, const
 SP_API int sp_window_attention(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kpool,
                                const void* vpool, const void* kpooled, const void* vpooled, int64_t kp_stride,
                                int64_t vp_stride, const int32_t* req_to_token, int64_t table_stride, int64_t num_tokens,
-                               int heads, int kv_heads, int dim, int vdim, int64_t window, int block, float scale,
-                               const float* sinks, float softcap, int sigmoid_weights, const float* head_bias,
+                               int heads, int kv_heads, int dim, int vdim, int64_t window, int block, int keep_first,
+                               float scale, const float* sinks, float softcap, int sigmoid_weights, const float* head_bias,
                                const void* gate, int64_t gate_stride, int matrix, SP_SEQ_PARAMS, int dtype, void* stream);
+/* (ABI 15) keep_first > 0 (without blocks): the tokens j < keep_first stay visible after they left the window.          */
 /* (ABI 13) softcap > 0: score = softcap tanh(score / softcap) after the scale.  sigmoid_weights != 0: no softmax - a
  * visible key's weight is sigmoid(score + head_bias[head]) (head_bias fp32 [heads], optional), not normalised; no sinks.
  * gate ([T, heads * vdim] in `dtype`, optional): the result is multiplied element by element with sigmoid(gate).        */
@@ -667,11 +683,36 @@ SP_API int sp_gated_delta_scan(void* out, int64_t out_stride, const void* q, int
  *   z null:  y = a
  *   else:    y = sum over k < top, in that order, of weights[t, k] * (ids[t, k] < experts ? z[place[t * top + k]] : x[t])
  *                + gate[t] * a[t]            (a optional; gate fp32 [T], optional: 1)
- * a, z [rows, width] in `dtype`, z contiguous.  width <= 15360.                                                         */
-SP_API int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a_stride, const void* z, const int32_t* ids,
-                        const int32_t* place, const float* weights, const float* gate, int experts, int top,
-                        const float* scale, float alpha, const float* weight, void* lo, int64_t lo_stride,
+ * a, z [rows, width] in `dtype`, z contiguous.  width <= 15360.
+ * (ABI 15) b (in `dtype`, with fp32 weights wa, wb [width]; not beside z): y = (N(a) wa + N(b) wb) / 2.                  */
+SP_API int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a_stride, const void* b, int64_t b_stride,
+                        const float* wa, const float* wb, const void* z, const int32_t* ids, const int32_t* place,
+                        const float* weights, const float* gate, int experts, int top, const float* scale, float alpha,
+                        const float* weight, void* lo, int64_t lo_stride,
                         int64_t num_tokens, int width, float eps, int dtype, void* stream);
+
+/* ================================================================================================================
+ * ABI 15: the head-gated delta rule and the tanh-GELU feed-forward (and sp_head_linear, positions in sp_embed_scale, branches
+ * in sp_post_norm, kept first tokens in sp_window_attention, epilogue 3 of sp_gemm_skinny, the matrix form of
+ * sp_latent_attention, all described at their place above).
+ */
+/* Per (request, value head h) over the request's rows of this step in order, S [dim, vdim] fp32 from state[request slot]
+ * (zeros at a sequence's first token) and back; query/key head h / (heads / kv_heads):
+ *   qn = q / sqrt(|q|^2 + 1e-6) dim^(-1/2);  kn = k / sqrt(|k|^2 + 1e-6);  beta = sigmoid(pre[t, h]);
+ *   g = exp(-exp(A_log[h]) softplus(pre[t, heads + h] + dt_bias[h]));  S = g S;  u = beta (v - S^T kn);  S = S + kn u^T;
+ *   o = S^T qn;  out = o / rms_head(o) * norm_w * silu(gate)
+ * q, k [T, kv_heads * dim], v, gate, out [T, heads * vdim] in `dtype`; pre fp32 [T, >= 2 heads]; norm_w fp32 [vdim].
+ * dim, vdim <= 256.  ranges > 1: that many workgroups share a head's value channels; they need the workspace (fp32,
+ * T * heads * vdim values).                                                                                            */
+SP_API int sp_head_delta_scan(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k, int64_t k_stride,
+                              const void* v, int64_t v_stride, const void* gate, int64_t gate_stride, const float* pre,
+                              int64_t pre_stride, const float* dt_bias, const float* A_log, const float* norm_w, float* state,
+                              int64_t state_stride, float* workspace, int64_t num_tokens, int heads, int kv_heads, int dim,
+                              int vdim, int ranges, float eps, SP_SEQ_PARAMS, int dtype, void* stream);
+/* out[t, j] = gelu_tanh(x[t, j]) * x[t, d + j], gelu_tanh(z) = z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))) in fp32, the
+ * product rounded once */
+SP_API int sp_gelu_tanh_and_mul(void* out, const void* x, int64_t num_tokens, int d, int64_t x_stride, int64_t out_stride,
+                                int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -116,9 +116,10 @@ SIGNATURES = {
     "sp_wkv_recurrence": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i64, _i64, _i64, _i64,
                                  _i64, _f32, *_SEQ, _i32, _vp]),
     "sp_rotary_interleaved": (_i32, [_vp, _vp, _vp, _f32, _i64, _i32, _i32, _i64, _i64, _i32, _i32, _vp]),
-    "sp_latent_kv_store": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _f32, _vp, _i64, _i32, _i32, _i32, _f32, _i32, _vp]),
-    "sp_latent_attention": (_i32, [_vp, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _i32, _i32, _i32, _i64, _i64, _f32, *_SEQ,
-                                   _i32, _vp]),
+    "sp_latent_kv_store": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _i64, _i64, _i32, _i32, _vp, _vp, _f32, _vp, _i64, _i32, _i32,
+                                  _i32, _f32, _i32, _vp]),
+    "sp_latent_attention": (_i32, [_vp, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64, _i64, _i32, _i32, _i32, _i64, _i64, _f32,
+                                   _i32, _i32, _vp, _i64, *_SEQ, _i32, _vp]),
     "sp_moe_route": (_i32, [_vp, _vp, _vp, _i64, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
     "sp_moe_align": (_i32, [_vp, _vp, _vp, _vp, _i32, _i32, _vp]),
     "sp_moe_grouped_gemm": (_i32, [_vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _i64, _i64, _i32, _i32, _vp]),
@@ -126,7 +127,7 @@ SIGNATURES = {
     "sp_moe_combine": (_i32, [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _i64, _i32, _vp]),
     # ---- ABI 11
     "sp_moe_softmax_topk": (_i32, [_vp, _vp, _vp, _vp, _i64, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
-    "sp_embed_scale": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _i64, _i32, _i64, _f32, _i32, _vp]),
+    "sp_embed_scale": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i64, _i32, _i64, _f32, _i32, _vp]),
     "sp_norm_shift": (_i32, [_vp, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _i64, _i32, _f32, *_SEQ, _i32, _vp]),
     "sp_norm_save_last": (_i32, [_vp, _i64, _vp, _i64, _vp, _i32, _f32, *_SEQ, _vp]),
     "sp_stream_add": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _i64, _i32, _i32, _vp]),
@@ -135,7 +136,7 @@ SIGNATURES = {
                                    _i64, _vp, _i32, _vp]),
     "sp_pool_blocks": (_i32, [_vp, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i32, _i32, _i32, *_SEQ, _i32, _vp]),
     "sp_window_attention": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i32, _i32, _i32,
-                                   _i32, _i64, _i32, _f32, _vp, _f32, _i32, _vp, _vp, _i64, _i32, *_SEQ, _i32, _vp]),
+                                   _i32, _i64, _i32, _i32, _f32, _vp, _f32, _i32, _vp, _vp, _i64, _i32, *_SEQ, _i32, _vp]),
     "sp_small_linear_f32": (_i32, [_vp, _vp, _i64, _vp, _vp, _i64, _i32, _i32, _i32, _vp]),
     "sp_causal_conv_silu": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _i64, _i32, _i32, *_SEQ, _i32, _vp]),
     "sp_mamba2_scan": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, *_SEQ, _i32, _vp]),
@@ -158,8 +159,13 @@ SIGNATURES = {
     "sp_gated_delta_scan": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _i32,
                                    _i32, _i32, _f32, *_SEQ, _i32, _vp]),
     # ---- ABI 14
-    "sp_post_norm": (_i32, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _vp, _f32, _vp, _vp, _i64, _i64, _i32,
+    "sp_post_norm": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _vp, _f32, _vp, _vp, _i64, _i64, _i32,
                             _f32, _i32, _vp]),
+    # ---- ABI 15
+    "sp_head_linear": (_i32, [_vp, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _i32, _vp]),
+    "sp_head_delta_scan": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64,
+                                  _vp, _i64, _i32, _i32, _i32, _i32, _i32, _f32, *_SEQ, _i32, _vp]),
+    "sp_gelu_tanh_and_mul": (_i32, [_vp, _vp, _i64, _i32, _i64, _i64, _i32, _vp]),
 }
 
 
@@ -193,7 +199,7 @@ def load() -> ctypes.CDLL:
             continue
         fn.restype = res
         fn.argtypes = args
-    if lib.sp_abi_version() != 14:
+    if lib.sp_abi_version() != 15:
         raise RuntimeError("libscratchpad_hip.so ABI version mismatch")
     _lib = lib
     return lib
@@ -287,6 +293,17 @@ def silu_and_mul(x: torch.Tensor) -> torch.Tensor:
     _check(load().sp_silu_and_mul(out.data_ptr(), x2.data_ptr(), x2.shape[0], d, x2.stride(0),
                                   out.stride(0), _dt(x), _stream()), "sp_silu_and_mul")
     return out.view(*x.shape[:-1], d)
+
+
+def gelu_tanh_and_mul(x: torch.Tensor) -> torch.Tensor:
+    """gelu_tanh(x[:, :d]) * x[:, d:] (the tanh form of GELU, fp32, the product rounded once)"""
+    if _mat(x, "x").shape[1] % 2:
+        raise RuntimeError("gelu_tanh_and_mul: x [T, 2 d]")
+    d = x.shape[1] // 2
+    out = empty_rows(x.shape[0], d, x.dtype, x.device)
+    _check(load().sp_gelu_tanh_and_mul(out.data_ptr(), x.data_ptr(), x.shape[0], d, x.stride(0), out.stride(0), _dt(x), _stream()),
+           "sp_gelu_tanh_and_mul")
+    return out
 
 
 def rotary_embedding(positions: torch.Tensor, query: torch.Tensor, key: torch.Tensor,
@@ -888,6 +905,17 @@ def linear_silu_mul(x: torch.Tensor, gate_up_weight: torch.Tensor, any_rows: boo
     SILU_FUSED_MAX_ROWS tokens (any_rows: up to the kernel's 16): x [M, K], gate_up_weight [2 I, K] (gate rows first),
     result [M, I].  Bit for bit the skinny projection followed by silu_and_mul.  None when the shape is not taken (the
     caller runs the two steps)."""
+    return _skinny_glu(x, gate_up_weight, any_rows, 1, "sp_gemm_skinny(silu)")
+
+
+def linear_gelu_mul(x: torch.Tensor, gate_up_weight: torch.Tensor) -> torch.Tensor:
+    """gelu_tanh(x @ gate.T) * (x @ up.T) of the merged matrix [gate | up]: one launch for a step of few tokens, the product and
+    gelu_tanh_and_mul one after the other elsewhere (the same bits)"""
+    out = _skinny_glu(x, gate_up_weight, False, 3, "sp_gemm_skinny(gelu)")
+    return gelu_tanh_and_mul(linear(x, gate_up_weight)) if out is None else out
+
+
+def _skinny_glu(x: torch.Tensor, gate_up_weight: torch.Tensor, any_rows: bool, epilogue: int, what: str) -> Optional[torch.Tensor]:
     if not (_SKINNY_ON and _SILU_LINEAR_ON and x.is_cuda and x.dim() == 2 and gate_up_weight.dim() == 2
             and 0 < x.shape[0] <= (SKINNY_MAX_ROWS if any_rows else SILU_FUSED_MAX_ROWS)
             and gate_up_weight.shape[1] == x.shape[1]
@@ -901,7 +929,7 @@ def linear_silu_mul(x: torch.Tensor, gate_up_weight: torch.Tensor, any_rows: boo
     inter = gate_up_weight.shape[0] // 2
     out = empty_rows(M, inter, x.dtype, x.device)
     _check(load().sp_gemm_skinny(out.data_ptr(), x.data_ptr(), gate_up_weight.data_ptr(), M, inter, K, x.stride(0),
-                                 gate_up_weight.stride(0), out.stride(0), 1, _dt(x), _stream()), "sp_gemm_skinny(silu)")
+                                 gate_up_weight.stride(0), out.stride(0), epilogue, _dt(x), _stream()), what)
     return out
 
 
@@ -1003,6 +1031,14 @@ class SeqParams:
 def _f32(t: torch.Tensor, what: str) -> torch.Tensor:
     if t.dtype != torch.float32 or not t.is_cuda or not t.is_contiguous():
         raise RuntimeError(f"{what} must be a contiguous fp32 device tensor")
+    return t
+
+
+def _heads(t: torch.Tensor, what: str) -> torch.Tensor:
+    """[T, H, n] with contiguous rows (any token and head stride)"""
+    _gpu(t)
+    if t.dim() != 3 or t.stride(2) != 1:
+        raise RuntimeError(f"{what} must be [T, H, n] with contiguous rows, got shape {tuple(t.shape)} strides {tuple(t.stride())}")
     return t
 
 
@@ -1146,32 +1182,89 @@ def rotary_interleaved(x: torch.Tensor, positions: torch.Tensor, freq: torch.Ten
 
 
 def latent_kv_store(pool: torch.Tensor, dkv: torch.Tensor, norm_w: torch.Tensor, positions: torch.Tensor,
-                    freq: torch.Tensor, mag: float, loc: torch.Tensor, rank: int, eps: float) -> None:
+                    freq: torch.Tensor, mag: float, loc: torch.Tensor, rank: int, eps: float,
+                    q: Optional[torch.Tensor] = None, q_offset: int = 0) -> None:
+    """pool[loc] = [normed latent | rotated key part] of dkv's rows; ``q`` [T, H, n] (a view) rotated in place at q_offset in
+    the same launch"""
     _mat(pool, "pool"), _mat(dkv, "dkv"), _f32(norm_w, "norm_w"), _f32(freq, "freq")
     rot_dim = dkv.shape[1] - rank
     if pool.dtype != dkv.dtype or pool.shape[1] != dkv.shape[1] or norm_w.shape[0] != rank or rot_dim < 2 * freq.shape[0] \
             or loc.dtype != torch.int64 or positions.dtype != torch.int64 or loc.shape[0] != dkv.shape[0]:
         raise RuntimeError("latent_kv_store: pool [P, rank + rot], dkv [T, rank + rot] of one dtype, int64 loc / positions")
-    _check(load().sp_latent_kv_store(pool.data_ptr(), pool.stride(0), dkv.data_ptr(), dkv.stride(0), norm_w.data_ptr(),
+    qs = (None, 0, 0, 0, 0)
+    if q is not None:
+        if _heads(q, "q").shape[0] != dkv.shape[0] or q.dtype != dkv.dtype or q_offset + 2 * freq.shape[0] > q.shape[2]:
+            raise RuntimeError("latent_kv_store: q [T, H, >= q_offset + rotated dims] of dkv's dtype")
+        qs = (q.data_ptr(), q.stride(0), q.stride(1), q_offset, q.shape[1])
+    _check(load().sp_latent_kv_store(pool.data_ptr(), pool.stride(0), dkv.data_ptr(), dkv.stride(0), norm_w.data_ptr(), *qs,
                                      positions.data_ptr(), freq.data_ptr(), mag, loc.data_ptr(), dkv.shape[0], rank, rot_dim,
                                      2 * freq.shape[0], eps, _dt(dkv), _stream()), "sp_latent_kv_store")
 
 
+def latent_rotate_query(q: torch.Tensor, positions: torch.Tensor, freq: torch.Tensor, mag: float, q_offset: int) -> None:
+    """the query half of latent_kv_store alone (a layer that reads another layer's rows)"""
+    _f32(freq, "freq")
+    dims = 2 * freq.shape[0]
+    if _heads(q, "q").shape[0] != positions.shape[0] or positions.dtype != torch.int64 or q_offset + dims > q.shape[2]:
+        raise RuntimeError("latent_rotate_query: q [T, H, >= q_offset + rotated dims], int64 positions")
+    _check(load().sp_latent_kv_store(None, 0, None, 0, None, q.data_ptr(), q.stride(0), q.stride(1), q_offset, q.shape[1],
+                                     positions.data_ptr(), freq.data_ptr(), mag, None, q.shape[0], 1, dims, dims, 0.0, _dt(q),
+                                     _stream()), "sp_latent_kv_store(query)")
+
+
+LATENT_WORKGROUPS = 512         # latent_attention shares keys out over workgroups until a launch has about this many
+LATENT_MAX_SPLITS = 32
+
+
+def latent_splits(rows: int, requests: int, decode: bool, max_keys: int) -> int:
+    """how many workgroups share the keys of one tile of query rows: rows = query rows (tokens x heads) of the step"""
+    per = rows // requests if decode else 64
+    block = 16 if per <= 16 else (32 if per <= 32 else 64)
+    tiles = requests * -(-per // block) if decode else -(-rows // block)
+    return max(1, min(LATENT_WORKGROUPS // max(tiles, 1), LATENT_MAX_SPLITS, -(-max_keys // 64)))
+
+
 def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, pool: torch.Tensor, req_to_token: torch.Tensor,
-                     seq: SeqParams, scale: float) -> torch.Tensor:
-    """q_lat [H, T, rank] contiguous; q_rot [T, H, rot] (a view: strides are taken); pool [P, rank + rot]; -> [H, T, rank]"""
+                     seq: SeqParams, scale: float, token_major: bool = False, matrix: bool = True,
+                     splits: Optional[int] = None) -> torch.Tensor:
+    """q_lat [H, T, rank] (``token_major``: [T, H, rank]) contiguous; q_rot [T, H, rot] (a view: strides are taken); pool
+    [P, rank + rot]; -> the shape of q_lat.  matrix=False keeps 16-bit steps off the matrix-core kernel (comparisons); splits:
+    how many workgroups share a query's keys there (None: by the step's size)."""
     _mat(pool, "pool")
-    H, T, rank = q_lat.shape
+    T, H, rank = q_lat.shape if token_major else (q_lat.shape[1], q_lat.shape[0], q_lat.shape[2])
     if not q_lat.is_contiguous() or q_rot.dim() != 3 or q_rot.stride(2) != 1 or q_rot.shape[:2] != (T, H) or \
             pool.shape[1] != rank + q_rot.shape[2] or q_lat.dtype != pool.dtype or q_rot.dtype != pool.dtype or \
             req_to_token.dtype != torch.int32 or T != seq.num_tokens:
         raise RuntimeError("latent_attention: shapes / dtypes do not fit")
-    out = torch.empty((H, T, rank), dtype=q_lat.dtype, device=q_lat.device)
-    _check(load().sp_latent_attention(out.data_ptr(), q_lat.data_ptr(), q_rot.data_ptr(), pool.data_ptr(), pool.stride(0),
+    out = torch.empty_like(q_lat)
+    ts, hs = (H * rank, rank) if token_major else (rank, T * rank)
+    if splits is None:
+        splits = latent_splits(T * H, seq.batch_size, seq.token_req is None, req_to_token.shape[1])
+    if q_lat.dtype == torch.float32 or not matrix:
+        splits = 1
+    ws = torch.empty(splits * T * H * (rank + 2), dtype=torch.float32, device=q_lat.device) if splits > 1 else None
+    _check(load().sp_latent_attention(out.data_ptr(), q_lat.data_ptr(), ts, hs, q_rot.data_ptr(), pool.data_ptr(), pool.stride(0),
                                       req_to_token.data_ptr(), req_to_token.stride(0), T, H, rank, q_rot.shape[2],
-                                      q_rot.stride(0), q_rot.stride(1), scale, *seq.args, _dt(q_lat), _stream()),
+                                      q_rot.stride(0), q_rot.stride(1), scale, int(matrix), splits, _ptr(ws),
+                                      0 if ws is None else ws.numel(), *seq.args, _dt(q_lat), _stream()),
            "sp_latent_attention")
     return out
+
+
+def head_linear(x: torch.Tensor, weight: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """[T, H, n]: out[t, h] = weight[h] x[t, h], x [T, H, k] (a view: strides are taken), weight [H, n, k]; ``gate`` [T, H * n]
+    (a view): the result times sigmoid(gate)"""
+    T, H, k = _heads(x, "x").shape
+    if weight.dim() != 3 or not weight.is_contiguous() or weight.shape[0] != H or weight.shape[2] != k or weight.dtype != x.dtype:
+        raise RuntimeError("head_linear: weight [H, n, k] contiguous, of x's dtype")
+    n = weight.shape[1]
+    if gate is not None and (_mat(gate, "gate").shape != (T, H * n) or gate.dtype != x.dtype):
+        raise RuntimeError("head_linear: gate [T, H * n] of x's dtype")
+    out = empty_rows(T, H * n, x.dtype, x.device)
+    _check(load().sp_head_linear(out.data_ptr(), out.stride(0), n, x.data_ptr(), x.stride(0), x.stride(1), weight.data_ptr(),
+                                 _ptr(gate), 0 if gate is None else gate.stride(0), T, H, n, k, _dt(x), _stream()),
+           "sp_head_linear")
+    return out.view(T, H, n)
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, correction: torch.Tensor, top: int, groups: int, keep: int):
@@ -1253,16 +1346,23 @@ def moe_route_softmax(x: torch.Tensor, router: torch.Tensor, top: int, scale: fl
     return (ids, weights, gate) if gate_row else (ids, weights)
 
 
-def embed_scale(embed: torch.Tensor, ids: torch.Tensor, scale: float, want_lo: bool = False):
-    """fp32 [T, W] = embed[ids] * scale; ``want_lo``: (that, the same in the table's dtype)"""
+def embed_scale(embed: torch.Tensor, ids: torch.Tensor, scale: float, want_lo: bool = False,
+                table: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None):
+    """fp32 [T, W] = embed[ids] * scale (+ table[positions], a learned row per position); ``want_lo``: (that, the same in the
+    table's dtype)"""
     _gpu(embed, ids)
+    if table is not None and (_gpu(table, positions) or positions.dtype != torch.int64 or positions.shape != ids.shape or
+                              table.dtype != embed.dtype or table.dim() != 2 or table.shape[1] != embed.shape[1] or
+                              not table.is_contiguous()):
+        raise RuntimeError("embed_scale: table [rows, width] contiguous, of embed's dtype, int64 positions")
     if ids.dtype != torch.int64 or embed.dim() != 2 or not embed.is_contiguous():
         raise RuntimeError("embed_scale: int64 ids, contiguous table [vocab, width]")
     x = torch.empty((ids.shape[0], embed.shape[1]), dtype=torch.float32, device=embed.device)
     lo = empty_rows(ids.shape[0], embed.shape[1], embed.dtype, embed.device) if want_lo else None
     _check(load().sp_embed_scale(x.data_ptr(), x.stride(0), _ptr(lo), 0 if lo is None else lo.stride(0), embed.data_ptr(),
-                                 ids.data_ptr(), ids.shape[0], embed.shape[1], embed.shape[0], scale, _dt(embed), _stream()),
-           "sp_embed_scale")
+                                 ids.data_ptr(), _ptr(table), _ptr(positions) if table is not None else None,
+                                 0 if table is None else table.shape[0], ids.shape[0], embed.shape[1], embed.shape[0], scale,
+                                 _dt(embed), _stream()), "sp_embed_scale")
     return (x, lo) if want_lo else x
 
 
@@ -1370,11 +1470,13 @@ def window_attention(q: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
                      vpooled: Optional[torch.Tensor], req_to_token: torch.Tensor, seq: SeqParams, heads: int, kv_heads: int,
                      dim: int, vdim: int, window: int, block: int, scale: float, matrix: bool = True,
                      sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, sigmoid_weights: bool = False,
-                     head_bias: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     head_bias: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                     keep_first: int = 0) -> torch.Tensor:
     """q [T, heads * dim] (rotated) -> [T, heads * vdim]; matrix=False keeps 16-bit prompt portions off the matrix-core
     kernel (comparisons); sinks fp32 [heads]: one more term exp(sink) in every softmax's denominator; softcap > 0: scores
     capped as softcap tanh(score / softcap); sigmoid_weights: a visible key's weight is sigmoid(score + head_bias[head]),
-    not normalised; gate [T, heads * vdim] (a view): the result times sigmoid(gate)"""
+    not normalised; gate [T, heads * vdim] (a view): the result times sigmoid(gate); keep_first: so many first tokens stay
+    visible behind the window (without blocks)"""
     _mat(q, "q"), _mat(kpool, "kpool"), _mat(vpool, "vpool")
     T = q.shape[0]
     if q.shape[1] != heads * dim or kpool.shape[1] != kv_heads * dim or vpool.shape[1] != kv_heads * vdim or \
@@ -1392,7 +1494,7 @@ def window_attention(q: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
     _check(load().sp_window_attention(out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), kpool.data_ptr(),
                                       vpool.data_ptr(), _ptr(kpooled), _ptr(vpooled), kpool.stride(0), vpool.stride(0),
                                       req_to_token.data_ptr(), req_to_token.stride(0), T, heads, kv_heads, dim, vdim,
-                                      window, block, scale, _ptr(sinks), float(softcap or 0.0), int(sigmoid_weights),
+                                      window, block, keep_first, scale, _ptr(sinks), float(softcap or 0.0), int(sigmoid_weights),
                                       _ptr(head_bias), _ptr(gate), 0 if gate is None else gate.stride(0), int(matrix),
                                       *seq.args, _dt(q), _stream()),
            "sp_window_attention")
@@ -1652,20 +1754,54 @@ def gated_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, bpre: to
     return out
 
 
+HEAD_DELTA_WORKGROUPS = 512     # a head's value channels are shared out until a launch has about this many workgroups
+
+
+def head_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, pre: torch.Tensor,
+                    dt_bias: torch.Tensor, A_log: torch.Tensor, norm_w: torch.Tensor, state: torch.Tensor, seq: SeqParams,
+                    heads: int, kv_heads: int, dim: int, vdim: int, eps: float, ranges: Optional[int] = None) -> torch.Tensor:
+    """q, k [T, kv_heads * dim], v, gate [T, heads * vdim] (views) -> [T, heads * vdim]; pre fp32 [T, 2 heads]: the
+    pre-activations of the step sizes, then of the decays; state [slots, heads, dim, vdim] fp32 is read and moved on.  ranges:
+    how many workgroups share a head's value channels (None: by the step's size)"""
+    T = seq.num_tokens
+    for name, t, w in (("q", q, kv_heads * dim), ("k", k, kv_heads * dim), ("v", v, heads * vdim), ("gate", gate, heads * vdim)):
+        if _mat(t, name).shape != (T, w) or t.dtype != q.dtype:
+            raise RuntimeError(f"head_delta_scan: {name} must be [num_tokens, {w}] of one dtype")
+    _f32(dt_bias, "dt_bias"), _f32(A_log, "A_log"), _f32(norm_w, "norm_w"), _f32(state, "state")
+    if _mat(pre, "pre").dtype != torch.float32 or pre.shape != (T, 2 * heads) or dt_bias.numel() != heads or \
+            A_log.numel() != heads or norm_w.numel() != vdim or state.shape[1:] != (heads, dim, vdim):
+        raise RuntimeError("head_delta_scan: pre fp32 [T, 2 H], dt_bias / A_log [H], norm_w [Dv], state [slots, H, D, Dv]")
+    if ranges is None:          # decode steps (one token per request) keep the norm and the gate in the scan
+        ranges = 1 if T <= seq.batch_size else max(1, min(HEAD_DELTA_WORKGROUPS // max(1, seq.batch_size * heads), vdim // 32))
+    out = empty_rows(T, heads * vdim, q.dtype, q.device)
+    ws = torch.empty(T * heads * vdim, dtype=torch.float32, device=q.device) if ranges > 1 else None
+    _check(load().sp_head_delta_scan(out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0),
+                                     v.data_ptr(), v.stride(0), gate.data_ptr(), gate.stride(0), pre.data_ptr(), pre.stride(0),
+                                     dt_bias.data_ptr(), A_log.data_ptr(), norm_w.data_ptr(), state.data_ptr(), state.stride(0),
+                                     _ptr(ws), T, heads, kv_heads, dim, vdim, ranges, eps, *seq.args, _dt(q), _stream()),
+           "sp_head_delta_scan")
+    return out
+
+
 # --------------------------------------------------------------------------- post-norm stream
 def post_norm(x: torch.Tensor, a: Optional[torch.Tensor], weight: torch.Tensor, eps: float, alpha: float, dtype: torch.dtype,
               scale: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
               place: Optional[torch.Tensor] = None, weights: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-              experts: int = 0, want_lo: bool = True) -> Optional[torch.Tensor]:
+              experts: int = 0, want_lo: bool = True, b: Optional[torch.Tensor] = None, wa: Optional[torch.Tensor] = None,
+              wb: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """x fp32 [T, W] = N(alpha x + scale * y) * weight in place; returns the new x in ``dtype`` (``want_lo``).  y = a, or with
     a mixture's rows z [T * top, W]: y[t] = sum_k weights[t, k] (z[place[t, k]], or x[t] itself where ids[t, k] >= experts)
-    + gate[t] a[t] (a optional, gate fp32 [T] or None: 1)."""
+    + gate[t] a[t] (a optional, gate fp32 [T] or None: 1); with a second branch b and weights wa, wb (fp32 [W]):
+    y = (N(a) wa + N(b) wb) / 2."""
     _mat(x, "x"), _f32(weight, "weight")
     T, W = x.shape
     if x.dtype != torch.float32 or weight.numel() != W or (scale is not None and _f32(scale, "scale").numel() != W):
         raise RuntimeError("post_norm: x fp32 [T, W], weight and scale [W]")
     if a is not None and (_mat(a, "a").shape != (T, W) or a.dtype != dtype):
         raise RuntimeError("post_norm: a must be [T, W] of the given dtype")
+    if b is not None and (a is None or z is not None or _mat(b, "b").shape != (T, W) or b.dtype != dtype or wa is None or
+                          wb is None or _f32(wa, "wa").numel() != W or _f32(wb, "wb").numel() != W):
+        raise RuntimeError("post_norm: two branches [T, W] of the given dtype with their weights wa, wb [W]")
     if z is None and (a is None or gate is not None):
         raise RuntimeError("post_norm: a result or a mixture's rows; a gate goes with the latter")
     top = 0
@@ -1677,7 +1813,8 @@ def post_norm(x: torch.Tensor, a: Optional[torch.Tensor], weight: torch.Tensor, 
                 (gate is not None and _f32(gate, "gate").numel() != T):
             raise RuntimeError("post_norm: z [T * top, W] contiguous, ids / weights [T, top], place [T * top], gate [T]")
     lo = empty_rows(T, W, dtype, x.device) if want_lo else None
-    _check(load().sp_post_norm(x.data_ptr(), x.stride(0), _ptr(a), 0 if a is None else a.stride(0), _ptr(z), _ptr(ids),
+    _check(load().sp_post_norm(x.data_ptr(), x.stride(0), _ptr(a), 0 if a is None else a.stride(0), _ptr(b),
+                               0 if b is None else b.stride(0), _ptr(wa), _ptr(wb), _ptr(z), _ptr(ids),
                                _ptr(place), _ptr(weights), _ptr(gate), experts, top, _ptr(scale), alpha, weight.data_ptr(),
                                _ptr(lo), 0 if lo is None else lo.stride(0), T, W, eps, _DTYPES[dtype], _stream()), "sp_post_norm")
     return lo

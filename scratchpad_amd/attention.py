@@ -528,15 +528,22 @@ class LatentAttention(nn.Module):
         self.scaling = scaling
         self.layer_id = layer_id
 
-    def forward(self, q_lat, q_rot, forward_batch: "ForwardBatch"):
-        """q_lat [H, T, rank], q_rot [T, H, rot_dim] (rotated) -> o_lat [H, T, rank]; the step's rows are in the pool"""
-        return forward_batch.attn_backend.forward_latent(q_lat, q_rot, self, forward_batch)
+    def store(self, dkv, norm_w, q, q_offset: int, rotary, positions, eps: float, forward_batch: "ForwardBatch") -> None:
+        """norm and rotate the step's rows dkv [T, rank + rot_dim] into the pool and rotate q [T, H, n] in place from
+        coordinate q_offset, in one launch; dkv None: the pool rows are another layer's, only q is rotated"""
+        forward_batch.attn_backend.store_latent(dkv, norm_w, q, q_offset, rotary, positions, eps, self, forward_batch)
+
+    def forward(self, q_lat, q_rot, forward_batch: "ForwardBatch", token_major: bool = False):
+        """q_lat [H, T, rank] (``token_major``: [T, H, rank]), q_rot [T, H, rot_dim] (rotated) -> o_lat in q_lat's shape; the
+        step's rows are in the pool"""
+        return forward_batch.attn_backend.forward_latent(q_lat, q_rot, self, forward_batch, token_major)
 
 
 class PooledWindowAttention(nn.Module):
     """Layer-local constants of a grouped-query attention layer over a WindowKVPool: a query sees the ``window`` latest
     tokens and, for every block of ``block`` positions wholly behind the window, the block's mean key and value (one
     softmax over both); key width ``dim`` and value width ``vdim`` may differ.  window None: plain causal attention.
+    ``keep_first``: so many first tokens of a sequence stay visible after they left the window (not beside blocks).
     ``sinks``: one learned fp32 number per query head whose exponential joins the softmax's denominator (a key every query
     sees, without a value).  ``norm_values``: the cache holds every value head divided by its root mean square.  q, k, v may
     carry fp32 biases (``store``), added before the rotation.
@@ -553,7 +560,7 @@ class PooledWindowAttention(nn.Module):
     def __init__(self, num_heads: int, num_kv_heads: int, dim: int, vdim: int, scaling: float, layer_id: int,
                  window: Optional[int] = None, block: Optional[int] = None, sinks: bool = False, norm_values: bool = True,
                  qk_norm=False, head_scale: bool = False, q_temp=None, softcap: float = 0.0,
-                 weights: str = "softmax", v_mix: bool = False, keys_as_values: bool = False):
+                 weights: str = "softmax", v_mix: bool = False, keys_as_values: bool = False, keep_first: int = 0):
         super().__init__()
         if num_heads % num_kv_heads:
             raise ValueError("query heads must be a multiple of key/value heads")
@@ -561,6 +568,9 @@ class PooledWindowAttention(nn.Module):
         self.dim, self.vdim, self.scaling, self.layer_id = dim, vdim, scaling, layer_id
         self.window = int(window) if window else 0
         self.block = int(block) if (block and window) else 0
+        self.keep_first = int(keep_first) if window else 0
+        if self.keep_first < 0 or (self.keep_first and self.block):
+            raise ValueError("kept first tokens and pooled blocks behind a window exclude each other")
         self.norm_values = norm_values
         if weights not in ("softmax", "sigmoid") or (weights == "sigmoid" and sinks):
             raise ValueError("weights: 'softmax' or 'sigmoid' (which has no sink)")
@@ -630,10 +640,18 @@ class SequenceBackend(AttentionBackend):
     def get_cuda_graph_seq_len_fill_value(self):
         return 1                  # a padded row is a sequence's first token on the reserved request row / dummy slot
 
-    def forward_latent(self, q_lat, q_rot, layer: LatentAttention, forward_batch: "ForwardBatch"):
+    def store_latent(self, dkv, norm_w, q, q_offset, rotary, positions, eps, layer: LatentAttention, forward_batch: "ForwardBatch"):
+        if dkv is None:
+            _native.latent_rotate_query(q, positions, rotary.freq, rotary.magnitude, q_offset)
+            return
+        pool = forward_batch.token_to_kv_pool.get_key_buffer(layer.layer_id)
+        _native.latent_kv_store(pool, dkv, norm_w, positions, rotary.freq, rotary.magnitude, forward_batch.out_cache_loc,
+                                layer.rank, eps, q=q, q_offset=q_offset)
+
+    def forward_latent(self, q_lat, q_rot, layer: LatentAttention, forward_batch: "ForwardBatch", token_major: bool = False):
         pool = forward_batch.token_to_kv_pool.get_key_buffer(layer.layer_id)
         return _native.latent_attention(q_lat, q_rot, pool, forward_batch.req_to_token_pool.req_to_token, self.seq,
-                                        layer.scaling)
+                                        layer.scaling, token_major=token_major)
 
     def store_window(self, q, k, v, rotary, positions, eps, layer: "PooledWindowAttention", forward_batch: "ForwardBatch",
                      cache_id=None, biases=(None, None, None), v_first_cache=None):
@@ -664,7 +682,8 @@ class SequenceBackend(AttentionBackend):
                                         layer.block, layer.scaling,
                                         sinks=None if layer.sinks is None else layer.sinks.data, softcap=layer.softcap,
                                         sigmoid_weights=layer.sigmoid_weights,
-                                        head_bias=None if layer.head_bias is None else layer.head_bias.data, gate=gate)
+                                        head_bias=None if layer.head_bias is None else layer.head_bias.data, gate=gate,
+                                        keep_first=layer.keep_first)
 
     def forward_decode(self, q, k, v, layer, forward_batch, save_kv_cache: bool = True):
         raise NotImplementedError("this backend serves latent attention layers (forward_latent) and windowed ones (forward_window)")

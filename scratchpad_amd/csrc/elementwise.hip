@@ -111,13 +111,18 @@ __global__ __launch_bounds__(kBlock) void rmsnorm_scalar_kernel(void* out,  // m
   }
 }
 
-// ------------------------------------------------------------------------------ SiLU-and-mul
+// ------------------------------------------------------------------------------ activation-and-mul
 // nn/layers/activation.py:22-24: F.silu(a) * b with both factors in `dtype` (silu rounded
 // before the product, as torch does).
-__device__ __forceinline__ float silu_f32(float a) { return silu_ref(a); }   // sp_common.h
+// ACT 1: gelu_tanh(a) * b, the product of two fp32 values rounded once.
+template <typename Tag, int ACT>
+__device__ __forceinline__ float glu_f32(float a, float b) {
+  if constexpr (ACT == 1) return __fmul_rn(gelu_tanh_f32(a), b);
+  else return __fmul_rn(Elem<Tag>::round(silu_ref(a)), b);   // sp_common.h
+}
 
-template <typename Tag>
-__global__ __launch_bounds__(kBlock) void silu_mul_vec_kernel(void* __restrict__ out,
+template <typename Tag, int ACT>
+__global__ __launch_bounds__(kBlock) void glu_mul_vec_kernel(void* __restrict__ out,
                                                                const void* __restrict__ x,
                                                                int64_t num_tokens, int d,
                                                                int64_t x_stride,
@@ -135,13 +140,13 @@ __global__ __launch_bounds__(kBlock) void silu_mul_vec_kernel(void* __restrict__
     unpack16<Tag>(ld16(row + (int64_t)v * 16), a);
     unpack16<Tag>(ld16(row + ((int64_t)d * E::kBytes) + (int64_t)v * 16), b);
 #pragma unroll
-    for (int e = 0; e < V; ++e) y[e] = __fmul_rn(E::round(silu_f32(a[e])), b[e]);
+    for (int e = 0; e < V; ++e) y[e] = glu_f32<Tag, ACT>(a[e], b[e]);
     st16((char*)out + t * o_stride * E::kBytes + (int64_t)v * 16, pack16<Tag>(y));
   }
 }
 
-template <typename Tag>
-__global__ __launch_bounds__(kBlock) void silu_mul_scalar_kernel(void* __restrict__ out,
+template <typename Tag, int ACT>
+__global__ __launch_bounds__(kBlock) void glu_mul_scalar_kernel(void* __restrict__ out,
                                                                   const void* __restrict__ x,
                                                                   int64_t num_tokens, int d,
                                                                   int64_t x_stride,
@@ -153,7 +158,7 @@ __global__ __launch_bounds__(kBlock) void silu_mul_scalar_kernel(void* __restric
     const int64_t t = i / d;
     const int j = (int)(i - t * d);
     const float a = E::load(x, t * x_stride + j), b = E::load(x, t * x_stride + d + j);
-    E::store(out, t * o_stride + j, __fmul_rn(E::round(silu_f32(a)), b));
+    E::store(out, t * o_stride + j, glu_f32<Tag, ACT>(a, b));
   }
 }
 
@@ -523,8 +528,8 @@ extern "C" int sp_fused_add_rmsnorm(void* x, void* residual, const void* weight,
                                                               (hipStream_t)stream)));
 }
 
-template <typename Tag>
-static int launch_silu(void* out, const void* x, int64_t T, int d, int64_t xs, int64_t os,
+template <typename Tag, int ACT>
+static int launch_glu(void* out, const void* x, int64_t T, int d, int64_t xs, int64_t os,
                        hipStream_t st) {
   typedef Elem<Tag> E;
   constexpr int V = E::kVec;
@@ -532,8 +537,8 @@ static int launch_silu(void* out, const void* x, int64_t T, int d, int64_t xs, i
   const int64_t work = vec ? T * (d / V) : T * (int64_t)d;
   int64_t blocks = (work + kBlock - 1) / kBlock;
   if (blocks > 256 * 16) blocks = 256 * 16;
-  if (vec) silu_mul_vec_kernel<Tag><<<dim3((unsigned)blocks), kBlock, 0, st>>>(out, x, T, d, xs, os);
-  else silu_mul_scalar_kernel<Tag><<<dim3((unsigned)blocks), kBlock, 0, st>>>(out, x, T, d, xs, os);
+  if (vec) glu_mul_vec_kernel<Tag, ACT><<<dim3((unsigned)blocks), kBlock, 0, st>>>(out, x, T, d, xs, os);
+  else glu_mul_scalar_kernel<Tag, ACT><<<dim3((unsigned)blocks), kBlock, 0, st>>>(out, x, T, d, xs, os);
   SP_LAUNCH_CHECK();
   return SP_OK;
 }
@@ -543,8 +548,17 @@ extern "C" int sp_silu_and_mul(void* out, const void* x, int64_t num_tokens, int
   SP_CHECK_ARG(num_tokens >= 0 && d > 0);
   if (num_tokens == 0) return SP_OK;
   SP_CHECK_ARG(out && x);
-  SP_DISPATCH_DTYPE(dtype, return (launch_silu<Tag>(out, x, num_tokens, d, x_stride, out_stride,
-                                                     (hipStream_t)stream)));
+  SP_DISPATCH_DTYPE(dtype, return (launch_glu<Tag, 0>(out, x, num_tokens, d, x_stride, out_stride,
+                                                       (hipStream_t)stream)));
+}
+
+extern "C" int sp_gelu_tanh_and_mul(void* out, const void* x, int64_t num_tokens, int d,
+                                    int64_t x_stride, int64_t out_stride, int dtype, void* stream) {
+  SP_CHECK_ARG(num_tokens >= 0 && d > 0);
+  if (num_tokens == 0) return SP_OK;
+  SP_CHECK_ARG(out && x && x_stride >= 2 * (int64_t)d && out_stride >= d);
+  SP_DISPATCH_DTYPE(dtype, return (launch_glu<Tag, 1>(out, x, num_tokens, d, x_stride, out_stride,
+                                                       (hipStream_t)stream)));
 }
 
 template <typename Tag>

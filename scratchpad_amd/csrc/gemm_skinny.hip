@@ -27,6 +27,8 @@
 // streams - was built first and measured 2 x SLOWER than the two launches: 76 vs 38 us at 1 row; the exponentials
 // of all 16 lane rows of every k-step are vector work the stream cannot hide.  profiles/NOTES.md, round 4.)
 // `epilogue` = 2: out = max(product, 0)^2 on the fp32 sum, rounded once (the up projection of a squared-ReLU feed-forward).
+// `epilogue` = 3: as 1 with the tanh form of GELU in SiLU's place, its product with the up sum rounded once (bit for bit the
+// plain projection followed by sp_gelu_tanh_and_mul).
 #include "sp_common.h"
 
 namespace sp {
@@ -68,22 +70,23 @@ constexpr int kSkWaves = 8;
 // gate_up 46.5 vs 43.3, LM head 186 vs 166; bench.py --bs 1: 4.13 vs 3.98 ms/step (round 3, tools/bench_gemv.py).
 __device__ __forceinline__ u32x4 ld16_nt(const void* p) { return __builtin_nontemporal_load((const u32x4*)p); }
 
-// EPI 1 (NB = 1 only): a.N = I output columns; the 16 W rows of a workgroup are gate rows n0 .. n0+7 (tile rows 0-7) and
+// EPI 1 and 3 (NB = 1 only): a.N = I output columns; the 16 W rows of a workgroup are gate rows n0 .. n0+7 (tile rows 0-7) and
 // up rows I + n0 .. I + n0 + 7 (tile rows 8-15)
 template <typename Tag, int NB, int UNROLL, bool NT, int EPI>
 __global__ __launch_bounds__(kSkWaves * 64) void gemm_skinny_kernel(SkinnyArgs a) {
   typedef Elem<Tag> E;
-  static_assert(EPI != 1 || NB == 1, "the SiLU-mul epilogue pairs the two halves of one 16-row tile");
+  constexpr bool GLU = EPI == 1 || EPI == 3;
+  static_assert(!GLU || NB == 1, "the activation-mul epilogue pairs the two halves of one 16-row tile");
   __shared__ float red[kSkWaves][NB][16 * 17];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r16 = lane & 15, q = lane >> 4;            // operand row / k-quarter of the lane
-  const int n0 = EPI == 1 ? blockIdx.x * 8 : blockIdx.x * 16 * NB;
+  const int n0 = GLU ? blockIdx.x * 8 : blockIdx.x * 16 * NB;
   const bool mrow = r16 < a.M;
   const char* wp[NB];
 #pragma unroll
   for (int nb = 0; nb < NB; ++nb) {
     int n = min(n0 + 16 * nb + r16, a.N - 1);          // clamp: columns past N are computed, never stored
-    if constexpr (EPI == 1) n = (r16 < 8 ? 0 : a.N) + min(n0 + (r16 & 7), a.N - 1);
+    if constexpr (GLU) n = (r16 < 8 ? 0 : a.N) + min(n0 + (r16 & 7), a.N - 1);
     wp[nb] = a.w + ((int64_t)n * a.w_stride + 8 * q) * 2;
   }
   const char* xp = a.x + ((int64_t)min(r16, a.M - 1) * a.x_stride + 8 * q) * 2;
@@ -127,15 +130,17 @@ __global__ __launch_bounds__(kSkWaves * 64) void gemm_skinny_kernel(SkinnyArgs a
       float s = 0.f;
 #pragma unroll
       for (int w = 0; w < kSkWaves; ++w) s += red[w][nb][col * 17 + r16];
-      if constexpr (EPI == 1) {
+      if constexpr (GLU) {
         // tile columns 0-7 are gate sums, 8-15 the up sums of the same output columns: the lanes of the gate half
-        // finish both (same summation order as above) and apply silu_mul_vec_kernel's arithmetic to the ROUNDED sums
+        // finish both (same summation order as above) and apply glu_mul_vec_kernel's arithmetic to the ROUNDED sums
         float su = 0.f;
 #pragma unroll
         for (int w = 0; w < kSkWaves; ++w) su += red[w][nb][((col & 7) + 8) * 17 + r16];
         const int n = n0 + col;
-        if (mrow && q < 2 && n < a.N)
-          E::store(a.out, (int64_t)r16 * a.out_stride + n, __fmul_rn(E::round(silu_ref(E::round(s))), E::round(su)));
+        if (mrow && q < 2 && n < a.N) {
+          const float act = EPI == 3 ? gelu_tanh_f32(E::round(s)) : E::round(silu_ref(E::round(s)));
+          E::store(a.out, (int64_t)r16 * a.out_stride + n, __fmul_rn(act, E::round(su)));
+        }
       } else {
         const int n = n0 + 16 * nb + col;
         if constexpr (EPI == 2) {
@@ -161,6 +166,7 @@ static void launch_skinny(const SkinnyArgs& a, int epilogue, hipStream_t st) {
   const bool u16 = g_skinny_u16 && (a.K / 32) % (16 * kSkWaves) == 0;
   if (epilogue == 1 && u16) gemm_skinny_kernel<Tag, 1, 16, false, 1><<<dim3((a.N + 7) / 8), block, 0, st>>>(a);
   else if (epilogue == 1) gemm_skinny_kernel<Tag, 1, 8, false, 1><<<dim3((a.N + 7) / 8), block, 0, st>>>(a);
+  else if (epilogue == 3) gemm_skinny_kernel<Tag, 1, 8, false, 3><<<dim3((a.N + 7) / 8), block, 0, st>>>(a);
   else if (epilogue == 2) gemm_skinny_kernel<Tag, 1, 8, false, 2><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
   else if (u16) gemm_skinny_kernel<Tag, 1, 16, false, 0><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
   else if (g_skinny_nt) gemm_skinny_kernel<Tag, 1, 8, true, 0><<<dim3((a.N + 15) / 16), block, 0, st>>>(a);
@@ -171,7 +177,7 @@ static void launch_skinny(const SkinnyArgs& a, int epilogue, hipStream_t st) {
 
 extern "C" int sp_gemm_skinny(void* out, const void* x, const void* w, int M, int N, int K, int64_t x_stride,
                               int64_t w_stride, int64_t out_stride, int epilogue, int dtype, void* stream) {
-  SP_CHECK_ARG(M >= 0 && N >= 0 && K > 0 && epilogue >= 0 && epilogue <= 2);
+  SP_CHECK_ARG(M >= 0 && N >= 0 && K > 0 && epilogue >= 0 && epilogue <= 3);
   if (M == 0 || N == 0) return SP_OK;
   SP_CHECK_ARG(out && x && w);
   if (M > 16 || K % 32 != 0) return SP_ERR_UNSUPPORTED;

@@ -2,11 +2,12 @@
 // latent c (rank C) from which every head's unrotated key W_uk c and value W_uv c derive, and the rotated key part
 // (R dimensions) all heads share.  The up-projections are folded into the query and the output:
 //   score(t, s, h) = (W_uk_h^T q_h[t]) . c[s] + q_rot_h[t] . k_rot[s]          out_h[t] = W_uv_h (sum_s p(t, s, h) c[s])
-// so the kernel is multi-query attention with key width C + R and value width C over the pool's rows; the caller
-// runs the two per-head products as batched matrix products around it.
+// so the kernel is multi-query attention with key width C + R and value width C over the pool's rows; the two per-head
+// products around it are sp_head_linear (out[t, h] = W_h x[t, h], optionally times sigmoid(gate)).
 //
 // Rotation: interleaved pairs (2i, 2i+1), angle = position * frequency[i] in fp32, cos and sin scaled by `mag`
-// (frequency table and magnitude are the caller's: plain, or YaRN-blended).
+// (frequency table and magnitude are the caller's: plain, or YaRN-blended).  The store can rotate the query's rotated part in
+// the same launch; a layer that reads another layer's rows only rotates its query.
 #include "seq_batch.h"
 
 namespace sp {
@@ -31,14 +32,36 @@ __global__ void rotary_interleaved_kernel(void* x, const int64_t* positions, con
   }
 }
 
-// pool[loc[t]] = [ rmsnorm(dkv[t, :C]) * w | rotate(dkv[t, C:C+R]) ]   (the first rot_dims of the R rotate, the rest pass)
+// pool[loc[t]] = [ rmsnorm(dkv[t, :C]) * w | rotate(dkv[t, C:C+R]) ]   (the first rot_dims of the R rotate, the rest pass);
+// q (optional): q[t, h, q_offset .. q_offset + rot_dims) rotated in place for every head.  The token's cosines and sines
+// (times mag) wait in LDS for all its heads.
+constexpr int kMaxRot = 512;
 template <typename Tag>
-__global__ void latent_kv_store_kernel(void* pool, int64_t pool_stride, const void* dkv, int64_t dkv_stride,
-                                       const float* norm_w, const int64_t* positions, const float* freq, float mag,
-                                       const int64_t* loc, int C, int R, int rot_dims, float eps) {
+__global__ void __launch_bounds__(kBlock)
+latent_kv_store_kernel(void* pool, int64_t pool_stride, const void* dkv, int64_t dkv_stride, const float* norm_w, void* q,
+                       int64_t q_stride, int64_t q_head_stride, int q_offset, int H, const int64_t* positions,
+                       const float* freq, float mag, const int64_t* loc, int C, int R, int rot_dims, float eps) {
   typedef Elem<Tag> E;
   __shared__ float red[kBlock / 64];
+  __shared__ float cosine[kMaxRot / 2], sine[kMaxRot / 2];
   const int64_t t = blockIdx.x;
+  const int half = rot_dims / 2;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
+    const float a = pos * freq[i];
+    cosine[i] = cosf(a) * mag;
+    sine[i] = sinf(a) * mag;
+  }
+  __syncthreads();
+  if (q)
+    for (int e = threadIdx.x; e < H * half; e += blockDim.x) {
+      const int h = e / half, i = e % half;
+      const int64_t at = t * q_stride + (int64_t)h * q_head_stride + q_offset + 2 * i;
+      const float u = E::load(q, at), v = E::load(q, at + 1);
+      E::store(q, at, u * cosine[i] - v * sine[i]);
+      E::store(q, at + 1, v * cosine[i] + u * sine[i]);
+    }
+  if (!pool) return;
   const int64_t src = t * dkv_stride, dst = loc[t] * pool_stride;
   float ss = 0.f;
   for (int i = threadIdx.x; i < C; i += blockDim.x) {
@@ -48,13 +71,10 @@ __global__ void latent_kv_store_kernel(void* pool, int64_t pool_stride, const vo
   ss = block_sum(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)C + eps);
   for (int i = threadIdx.x; i < C; i += blockDim.x) E::store(pool, dst + i, E::load(dkv, src + i) * inv * norm_w[i]);
-  const float pos = (float)positions[t];
-  for (int i = threadIdx.x; i < rot_dims / 2; i += blockDim.x) {
-    const float a = pos * freq[i];
-    const float c = cosf(a) * mag, s = sinf(a) * mag;
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
     const float u = E::load(dkv, src + C + 2 * i), v = E::load(dkv, src + C + 2 * i + 1);
-    E::store(pool, dst + C + 2 * i, u * c - v * s);
-    E::store(pool, dst + C + 2 * i + 1, v * c + u * s);
+    E::store(pool, dst + C + 2 * i, u * cosine[i] - v * sine[i]);
+    E::store(pool, dst + C + 2 * i + 1, v * cosine[i] + u * sine[i]);
   }
   for (int i = rot_dims + threadIdx.x; i < R; i += blockDim.x) E::store(pool, dst + C + i, E::load(dkv, src + C + i));
 }
@@ -65,9 +85,9 @@ constexpr int kMaxPerLane = 16;      // value width C <= 64 * kMaxPerLane
 // lane = value channel for the weighted sum; running maximum and sum in fp32.
 template <typename Tag>
 __global__ void __launch_bounds__(256)
-latent_attention_kernel(void* out, const void* q_lat, const void* q_rot, const void* pool, int64_t pool_stride,
-                        const int32_t* req_to_token, int64_t table_stride, SeqBatch s, int64_t T, int H, int C, int R,
-                        int64_t qrot_token_stride, int64_t qrot_head_stride, float scale) {
+latent_attention_kernel(void* out, const void* q_lat, int64_t lat_token_stride, int64_t lat_head_stride, const void* q_rot,
+                        const void* pool, int64_t pool_stride, const int32_t* req_to_token, int64_t table_stride, SeqBatch s,
+                        int64_t T, int H, int C, int R, int64_t qrot_token_stride, int64_t qrot_head_stride, float scale) {
   typedef Elem<Tag> E;
   extern __shared__ float smem[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -81,7 +101,7 @@ latent_attention_kernel(void* out, const void* q_lat, const void* q_rot, const v
   seq_of_token(s, t, b, start, prefix);
   const int64_t keys = prefix + (t - start) + 1;        // positions 0 .. own
   const int32_t* table = req_to_token + load_idx(s.req_pool_indices, b, s.idx64) * table_stride;
-  for (int i = lane; i < C; i += 64) sq[i] = E::load(q_lat, ((int64_t)h * T + t) * C + i) * scale;
+  for (int i = lane; i < C; i += 64) sq[i] = E::load(q_lat, t * lat_token_stride + h * lat_head_stride + i) * scale;
   for (int i = lane; i < R; i += 64) sq[C + i] = E::load(q_rot, t * qrot_token_stride + (int64_t)h * qrot_head_stride + i) * scale;
   __builtin_amdgcn_wave_barrier();
   float m = -INFINITY, l = 0.f;
@@ -126,7 +146,466 @@ latent_attention_kernel(void* out, const void* q_lat, const void* q_rot, const v
 #pragma unroll
   for (int i = 0; i < kMaxPerLane; ++i) {
     const int c = lane + 64 * i;
-    if (c < C) E::store(out, ((int64_t)h * T + t) * C + c, acc[i] * inv);
+    if (c < C) E::store(out, t * lat_token_stride + h * lat_head_stride + c, acc[i] * inv);
+  }
+}
+
+// ---- the same attention on the matrix cores, for 16-bit types -------------------------------------------------------
+// All heads of a token read the same pool rows, so the queries of one request are ONE list of rows (token-major, then head)
+// whatever the head count.  A workgroup of 4 waves takes RB blocks of 16 such rows and walks the keys they can see in tiles
+// of 64, staged in LDS row by row (the next tile's rows are in flight during the work on this one):
+//   S^T = K Q^T   v_mfma_f32_16x16x32, first operand = 16 key rows from LDS, second = the query fragments, in registers for
+//                 the whole walk: wave w forms KBW of the tile's 4 key blocks for RBW of the RB row blocks.  A lane receives
+//                 four keys of ONE query; a query's maximum is a reduction over its lanes and, through LDS, over the waves.
+//   P             exp of the scores, as a 16-bit value plus its 16-bit remainder (the weights are never rounded to 8 bits
+//                 of mantissa), goes to LDS in exactly the register layout the second product wants.
+//   O^T = V^T P^T the value is the first C columns of the same rows: its transposed fragments come from the key tile by
+//                 transposing LDS reads.  Wave w owns the value channels [16 DTW w, 16 DTW (w + 1)) of all RB row blocks.
+// With splits > 1 the tiles of a row block are shared out over blockIdx.y; every share writes its unnormalised sum, maximum
+// and denominator, and latent_merge_kernel joins them in the order of the keys (decode steps: few rows, many keys).
+typedef float f32x4_l __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x8_l __attribute__((ext_vector_type(8)));
+typedef _Float16 f16x8_l __attribute__((ext_vector_type(8)));
+typedef short s16x4_l __attribute__((ext_vector_type(4)));
+template <typename Tag>
+__device__ __forceinline__ f32x4_l mfma_l(const u32x4& a, const u32x4& b, const f32x4_l& c);
+template <>
+__device__ __forceinline__ f32x4_l mfma_l<bf16_tag>(const u32x4& a, const u32x4& b, const f32x4_l& c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_l, a), __builtin_bit_cast(bf16x8_l, b), c, 0, 0, 0);
+}
+template <>
+__device__ __forceinline__ f32x4_l mfma_l<f16_tag>(const u32x4& a, const u32x4& b, const f32x4_l& c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8_l, a), __builtin_bit_cast(f16x8_l, b), c, 0, 0, 0);
+}
+
+struct LatentArgs {
+  void* out;
+  const void* q_lat;
+  const void* q_rot;
+  const void* pool;
+  const int32_t* req_to_token;
+  float* part;                 // splits > 1: [splits][T * H][C] sums, then [splits][T * H][2] maximum and denominator
+  int64_t lat_token_stride, lat_head_stride, qrot_token_stride, qrot_head_stride, pool_stride, table_stride, T;
+  int H, C, R, splits;
+  float scale;
+};
+
+constexpr int kKeyTile = 64;
+template <int KS>
+constexpr int key_row() { return 32 * KS + 8; }      // elements per LDS row: 16 bytes of padding spread the rows over the banks
+template <int KS, int RB>
+constexpr size_t latent_lds() {
+  return (size_t)kKeyTile * key_row<KS>() * 2 + (size_t)RB * 4096 + (4 * 2 * 16 + RB * 16 + 4 * 2 * 16) * sizeof(float);
+}
+
+template <typename Tag, int KS, int DTW, int RB>
+__global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBatch s) {
+  typedef Elem<Tag> E;
+  constexpr int RBW = RB > 1 ? 2 : 1;                 // row blocks a wave scores
+  constexpr int GROUPS = RB / RBW;                    // groups of row blocks
+  constexpr int KBW = GROUPS;                         // key blocks (of 4) a wave scores: GROUPS * (4 / KBW) = 4 waves
+  constexpr int KR = key_row<KS>();
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  uint16_t* sk = (uint16_t*)lds;                                       // [64][KR]
+  u32x2* sp_ = (u32x2*)(lds + (size_t)kKeyTile * KR * 2);              // [RB][2][4 key blocks][64 lanes]
+  float* smax = (float*)(lds + (size_t)kKeyTile * KR * 2 + RB * 4096); // [4 waves][RBW][16]
+  float* scorr = smax + 4 * 2 * 16;                                    // [RB][16]
+  float* ssum = scorr + RB * 16;                                       // [4 waves][RBW][16]
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
+  const int rg = wave % GROUPS, kg = wave / GROUPS;
+  // which request and which of its row tiles
+  int64_t start, len, prefix;
+  int tile = blockIdx.x, b = 0;
+  if (s.extend_seq_lens) {
+    for (; b < s.B; ++b) {
+      const int tiles = (int)(((int64_t)s.extend_seq_lens[b] * a.H + 16 * RB - 1) / (16 * RB));
+      if (tile < tiles) {
+        tile = tiles - 1 - tile;                                       // the tiles with most keys start first
+        break;
+      }
+      tile -= tiles;
+    }
+    if (b >= s.B) return;
+  } else {
+    const int tiles = (a.H + 16 * RB - 1) / (16 * RB);
+    b = tile / tiles;
+    tile = tile % tiles;
+    if (b >= s.B) return;
+  }
+  seq_span(s, b, start, len, prefix);
+  const int64_t row0 = (int64_t)tile * 16 * RB, rows = len * a.H;      // rows of this request, this tile's first
+  const int64_t last_row = row0 + 16 * RB <= rows ? row0 + 16 * RB - 1 : rows - 1;
+  const int64_t keys = prefix + last_row / a.H + 1;
+  const int64_t tiles_k = (keys + kKeyTile - 1) / kKeyTile;
+  const int64_t per = (tiles_k + a.splits - 1) / a.splits;
+  const int64_t kt0 = (int64_t)blockIdx.y * per, kt1 = kt0 + per < tiles_k ? kt0 + per : tiles_k;
+  const int32_t* table = a.req_to_token + load_idx(s.req_pool_indices, b, s.idx64) * a.table_stride;
+  const int chunks = (a.C + a.R) / 8;                                  // 16-byte pieces of a pool row
+  // this lane's query rows (column r16 of every S^T block): fragments and the last key each may see
+  u32x4 qf[RBW][KS];
+  int64_t qpos[RBW];
+#pragma unroll
+  for (int i = 0; i < RBW; ++i) {
+    const int64_t r = row0 + 16 * (rg * RBW + i) + r16;
+    const bool on = r < rows;
+    const int64_t t = start + (on ? r / a.H : 0), h = on ? r % a.H : 0;
+    qpos[i] = on ? prefix + (t - start) : -1;
+#pragma unroll
+    for (int st = 0; st < KS; ++st) {
+      const int k = 32 * st + 8 * qd;
+      u32x4 f = {0u, 0u, 0u, 0u};
+      if (on && k < a.C) f = ld16((const char*)a.q_lat + (t * a.lat_token_stride + h * a.lat_head_stride + k) * 2);
+      else if (on && k < a.C + a.R) f = ld16((const char*)a.q_rot + (t * a.qrot_token_stride + h * a.qrot_head_stride + k - a.C) * 2);
+      qf[i][st] = f;
+    }
+  }
+  // columns behind the row are zero in every tile
+  for (int e = threadIdx.x; e < kKeyTile * (4 * KS - chunks); e += 256) {
+    const int n = 4 * KS - chunks, key = e / n, c = chunks + e % n;
+    st16((char*)(sk + key * KR + 8 * c), u32x4{0u, 0u, 0u, 0u});
+  }
+  f32x4_l oacc[DTW][RB];
+#pragma unroll
+  for (int d = 0; d < DTW; ++d)
+#pragma unroll
+    for (int i = 0; i < RB; ++i) oacc[d][i] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+  float m[RBW], l[RBW];
+#pragma unroll
+  for (int i = 0; i < RBW; ++i) {
+    m[i] = -INFINITY;
+    l[i] = 0.f;
+  }
+  // 16-byte pieces this thread moves per tile: threadIdx.x + 256 u
+  const int dk = 256 / chunks, dc = 256 % chunks, key_first = threadIdx.x / chunks, c_first = threadIdx.x % chunks;
+  u32x4 stage[KS];
+  auto fetch = [&](int64_t kt) {
+    int key = key_first, c = c_first;
+#pragma unroll
+    for (int u = 0; u < KS; ++u) {
+      const int64_t kk = kt * kKeyTile + key;
+      stage[u] = u32x4{0u, 0u, 0u, 0u};
+      if (key < kKeyTile && kk < keys) stage[u] = ld16((const char*)a.pool + ((int64_t)table[kk] * a.pool_stride + 8 * c) * 2);
+      key += dk;
+      c += dc;
+      if (c >= chunks) {
+        c -= chunks;
+        ++key;
+      }
+    }
+  };
+  if (kt0 < kt1) fetch(kt0);
+  for (int64_t kt = kt0; kt < kt1; ++kt) {
+    __syncthreads();                                                   // the previous tile's readers are done
+    {
+      int key = key_first, c = c_first;
+#pragma unroll
+      for (int u = 0; u < KS; ++u) {
+        if (key < kKeyTile) st16((char*)(sk + key * KR + 8 * c), stage[u]);
+        key += dk;
+        c += dc;
+        if (c >= chunks) {
+          c -= chunks;
+          ++key;
+        }
+      }
+    }
+    __syncthreads();
+    if (kt + 1 < kt1) fetch(kt + 1);
+    f32x4_l sacc[RBW][KBW];
+#pragma unroll
+    for (int i = 0; i < RBW; ++i)
+#pragma unroll
+      for (int j = 0; j < KBW; ++j) sacc[i][j] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int st = 0; st < KS; ++st)
+#pragma unroll
+      for (int j = 0; j < KBW; ++j) {
+        const u32x4 kf = ld16((const char*)(sk + (16 * (kg * KBW + j) + r16) * KR + 32 * st + 8 * qd));
+#pragma unroll
+        for (int i = 0; i < RBW; ++i) sacc[i][j] = mfma_l<Tag>(kf, qf[i][st], sacc[i][j]);
+      }
+    float mx[RBW];
+#pragma unroll
+    for (int i = 0; i < RBW; ++i) {
+      mx[i] = -INFINITY;
+#pragma unroll
+      for (int j = 0; j < KBW; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int64_t kk = kt * kKeyTile + 16 * (kg * KBW + j) + 4 * qd + r;
+          const float v = kk <= qpos[i] ? sacc[i][j][r] * a.scale : -INFINITY;
+          sacc[i][j][r] = v;
+          mx[i] = fmaxf(mx[i], v);
+        }
+      mx[i] = fmaxf(mx[i], __shfl_xor(mx[i], 16, 64));
+      mx[i] = fmaxf(mx[i], __shfl_xor(mx[i], 32, 64));
+      if (qd == 0) smax[(wave * RBW + i) * 16 + r16] = mx[i];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < RBW; ++i) {
+      float m_new = m[i];
+#pragma unroll
+      for (int w = rg; w < 4; w += GROUPS) m_new = fmaxf(m_new, smax[(w * RBW + i) * 16 + r16]);
+      const float m_safe = m_new == -INFINITY ? 0.f : m_new;           // nothing seen yet: every weight is exp(-inf) = 0
+      const float corr = expf(m[i] - m_safe);
+      m[i] = m_new;
+      float psum = 0.f;
+#pragma unroll
+      for (int j = 0; j < KBW; ++j) {
+        float p[8], rest[8], back[8];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          p[r] = expf(sacc[i][j][r] - m_safe);
+          psum += p[r];
+          p[4 + r] = 0.f;
+        }
+        const u32x4 hi = pack16<Tag>(p);
+        unpack16<Tag>(hi, back);
+#pragma unroll
+        for (int r = 0; r < 8; ++r) rest[r] = p[r] - back[r];
+        const u32x4 lo = pack16<Tag>(rest);
+        u32x2* at = sp_ + ((rg * RBW + i) * 8 + kg * KBW + j) * 64 + lane;
+        at[0] = u32x2{hi[0], hi[1]};
+        at[4 * 64] = u32x2{lo[0], lo[1]};
+      }
+      l[i] = l[i] * corr + psum;                                       // this lane's keys only: joined at the end
+      if (kg == 0 && qd == 0) scorr[(rg * RBW + i) * 16 + r16] = corr;
+    }
+    __syncthreads();
+    float cr[RB];
+#pragma unroll
+    for (int i = 0; i < RB; ++i) cr[i] = scorr[i * 16 + r16];
+#pragma unroll
+    for (int d = 0; d < DTW; ++d)
+#pragma unroll
+      for (int i = 0; i < RB; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) oacc[d][i][r] *= cr[i];
+#pragma unroll
+    for (int hh = 0; hh < 2; ++hh) {
+      u32x4 ph[RB], pl[RB];
+#pragma unroll
+      for (int i = 0; i < RB; ++i) {
+        const u32x2* at = sp_ + (i * 8 + 2 * hh) * 64 + lane;
+        const u32x2 h0 = at[0], h1 = at[64], l0 = at[256], l1 = at[320];
+        ph[i] = u32x4{h0[0], h0[1], h1[0], h1[1]};
+        pl[i] = u32x4{l0[0], l0[1], l1[0], l1[1]};
+      }
+#pragma unroll
+      for (int d = 0; d < DTW; ++d) {
+        const int ch = 16 * (wave * DTW + d);
+        if (ch >= a.C) continue;                                       // (the same for the whole wave)
+        // lane i of a 16-lane group addresses row 4 qd + (i >> 2), elements 4 (i & 3) .. + 3, and receives column i
+        const uint16_t* vp = sk + (32 * hh + 4 * qd + (r16 >> 2)) * KR + ch + 4 * (r16 & 3);
+        const u32x2 v0 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                                                       (__attribute__((address_space(3))) s16x4_l*)vp));
+        const u32x2 v1 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                                                       (__attribute__((address_space(3))) s16x4_l*)(vp + 16 * KR)));
+        const u32x4 vf = {v0[0], v0[1], v1[0], v1[1]};
+#pragma unroll
+        for (int i = 0; i < RB; ++i) {
+          oacc[d][i] = mfma_l<Tag>(vf, ph[i], oacc[d][i]);
+          oacc[d][i] = mfma_l<Tag>(vf, pl[i], oacc[d][i]);
+        }
+      }
+    }
+  }
+  // denominators: over the lanes of a query, then over the waves that scored its keys
+#pragma unroll
+  for (int i = 0; i < RBW; ++i) {
+    l[i] += __shfl_xor(l[i], 16, 64);
+    l[i] += __shfl_xor(l[i], 32, 64);
+    if (qd == 0) ssum[(wave * RBW + i) * 16 + r16] = l[i];
+  }
+  __syncthreads();
+  float inv[RB];
+#pragma unroll
+  for (int i = 0; i < RB; ++i) {
+    float den = 0.f;
+#pragma unroll
+    for (int w = i / RBW; w < 4; w += GROUPS) den += ssum[(w * RBW + i % RBW) * 16 + r16];
+    inv[i] = den;
+  }
+  if (a.splits > 1 && kg == 0 && qd == 0) {
+    float* ml = a.part + (int64_t)a.splits * a.T * a.H * a.C;
+#pragma unroll
+    for (int i = 0; i < RBW; ++i) {
+      const int64_t r = row0 + 16 * (rg * RBW + i) + r16;
+      if (r < rows) {
+        float* at = ml + ((int64_t)blockIdx.y * a.T * a.H + start * a.H + r) * 2;
+        at[0] = m[i];
+        at[1] = inv[rg * RBW + i];
+      }
+    }
+  }
+  if (a.splits > 1 && kt0 >= kt1) return;                              // no keys: the merge skips this share
+#pragma unroll
+  for (int i = 0; i < RB; ++i) {
+    const int64_t r = row0 + 16 * i + r16;
+    if (r >= rows) continue;
+    const int64_t t = start + r / a.H, h = r % a.H;
+    const float sc = a.splits > 1 ? 1.f : 1.f / inv[i];
+#pragma unroll
+    for (int d = 0; d < DTW; ++d) {
+      const int ch = 16 * (wave * DTW + d) + 4 * qd;
+      if (ch >= a.C) continue;
+      float f[8] = {oacc[d][i][0] * sc, oacc[d][i][1] * sc, oacc[d][i][2] * sc, oacc[d][i][3] * sc, 0.f, 0.f, 0.f, 0.f};
+      if (a.splits > 1) {
+        st16(a.part + ((int64_t)blockIdx.y * a.T * a.H + start * a.H + r) * a.C + ch, pack16<f32_tag>(f));
+      } else {
+        const u32x4 pk = pack16<Tag>(f);
+        *(u32x2*)((char*)a.out + (t * a.lat_token_stride + h * a.lat_head_stride + ch) * 2) = u32x2{pk[0], pk[1]};
+      }
+    }
+  }
+}
+
+// one workgroup per row: the shares' sums joined in the order of the keys
+template <typename Tag>
+__global__ void __launch_bounds__(128) latent_merge_kernel(LatentArgs a) {
+  typedef Elem<Tag> E;
+  const int64_t r = blockIdx.x, n = a.T * a.H, t = r / a.H, h = r % a.H;
+  const float* ml = a.part + (int64_t)a.splits * n * a.C;
+  float M = -INFINITY;
+  for (int s = 0; s < a.splits; ++s) M = fmaxf(M, ml[((int64_t)s * n + r) * 2]);      // (a row has seen itself: M is finite)
+  float den = 0.f;
+  for (int s = 0; s < a.splits; ++s) den += ml[((int64_t)s * n + r) * 2 + 1] * expf(ml[((int64_t)s * n + r) * 2] - M);
+  const float inv = 1.f / den;
+  for (int c = 4 * threadIdx.x; c < a.C; c += 512) {
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < a.splits; ++s) {
+      const float w = expf(ml[((int64_t)s * n + r) * 2] - M);
+      if (w == 0.f) continue;                                          // a share without keys has written no sum
+      float f[4];
+      unpack16<f32_tag>(ld16(a.part + ((int64_t)s * n + r) * a.C + c), f);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc[e] += w * f[e];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) acc[e] *= inv;
+    const u32x4 pk = pack16<Tag>(acc);
+    *(u32x2*)((char*)a.out + (t * a.lat_token_stride + h * a.lat_head_stride + c) * 2) = u32x2{pk[0], pk[1]};
+  }
+}
+
+template <typename Tag, int KS, int DTW, int RB>
+static int launch_latent_mfma(const LatentArgs& a, const SeqBatch& s, hipStream_t st) {
+  constexpr size_t lds = latent_lds<KS, RB>();
+  if (lds > 64 * 1024) {         // the limit is the device's: raised once per device of the process
+    static PerDevice<int> raised;
+    int ok = 0;
+    raised.get(ok, [&](int) {
+      return hipFuncSetAttribute((const void*)latent_mfma_kernel<Tag, KS, DTW, RB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                 (int)lds) == hipSuccess ? 1 : 0;
+    });
+    if (!ok) return SP_ERR_LAUNCH;
+  }
+  const int64_t blocks = s.extend_seq_lens ? (a.T * a.H + 16 * RB - 1) / (16 * RB) + s.B
+                                           : (int64_t)s.B * ((a.H + 16 * RB - 1) / (16 * RB));
+  latent_mfma_kernel<Tag, KS, DTW, RB><<<dim3((unsigned)blocks, (unsigned)a.splits), 256, lds, st>>>(a, s);
+  SP_LAUNCH_CHECK();
+  if (a.splits > 1) {
+    latent_merge_kernel<Tag><<<dim3((unsigned)(a.T * a.H)), 128, 0, st>>>(a);
+    SP_LAUNCH_CHECK();
+  }
+  return SP_OK;
+}
+template <typename Tag, int KS, int DTW>
+static int launch_latent_rows(const LatentArgs& a, const SeqBatch& s, hipStream_t st) {
+  const int64_t rows = s.extend_seq_lens ? 64 : a.H;                   // rows a request brings in a decode step
+  if (rows <= 16) return launch_latent_mfma<Tag, KS, DTW, 1>(a, s, st);
+  if (rows <= 32) return launch_latent_mfma<Tag, KS, DTW, 2>(a, s, st);
+  return launch_latent_mfma<Tag, KS, DTW, 4>(a, s, st);
+}
+template <typename Tag>
+static int launch_latent(const LatentArgs& a, const SeqBatch& s, hipStream_t st) {
+  if (a.C + a.R <= 160 && a.C <= 128) return launch_latent_rows<Tag, 5, 2>(a, s, st);
+  if (a.C + a.R <= 320 && a.C <= 256) return launch_latent_rows<Tag, 10, 4>(a, s, st);
+  if (a.C + a.R <= 576 && a.C <= 512) return launch_latent_rows<Tag, 18, 8>(a, s, st);
+  return SP_ERR_UNSUPPORTED;
+}
+
+// ---- out[t, h, n] = sum_k w[h, n, k] x[t, h, k]  (times sigmoid(gate[t, h N + n])) ---------------------------------------
+// 16-bit: a wave forms TT x NT tiles of 16 tokens x 16 outputs of one head, operands straight from memory (a head's matrix is
+// small and stays in the L2); TW of the 4 waves lie along the tokens, the others along the outputs.
+template <typename Tag, int TT, int NT, int TW>
+__global__ void __launch_bounds__(256)
+head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const void* x, int64_t x_stride, int64_t x_head,
+                        const void* w, const void* gate, int64_t gate_stride, int64_t T, int N, int K) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
+  const int64_t h = blockIdx.z;
+  const int64_t t0 = ((int64_t)blockIdx.x * TW + wave % TW) * (16 * TT);
+  const int n0 = (blockIdx.y * (4 / TW) + wave / TW) * (16 * NT);
+  if (t0 >= T || n0 >= N) return;                                      // (no workgroup barrier below)
+  const char *xp[TT], *wp[NT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    const int64_t t = t0 + 16 * i + r16 < T ? t0 + 16 * i + r16 : T - 1;
+    xp[i] = (const char*)x + (t * x_stride + h * x_head + 8 * qd) * 2;
+  }
+#pragma unroll
+  for (int j = 0; j < NT; ++j) {
+    const int n = n0 + 16 * j + r16 < N ? n0 + 16 * j + r16 : N - 1;
+    wp[j] = (const char*)w + ((h * N + n) * (int64_t)K + 8 * qd) * 2;
+  }
+  f32x4_l acc[TT][NT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int k = 0; k < K; k += 32) {
+    const bool on = k + 8 * qd < K;                                    // K is a multiple of 8
+    u32x4 xf[TT], wf[NT];
+#pragma unroll
+    for (int i = 0; i < TT; ++i) xf[i] = on ? ld16(xp[i] + 2 * k) : u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int j = 0; j < NT; ++j) wf[j] = on ? ld16(wp[j] + 2 * k) : u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int i = 0; i < TT; ++i)
+#pragma unroll
+      for (int j = 0; j < NT; ++j) acc[i][j] = mfma_l<Tag>(wf[j], xf[i], acc[i][j]);
+  }
+  // acc[i][j][r] = out[t0 + 16 i + r16][n0 + 16 j + 4 qd + r]; N is a multiple of 4
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    const int64_t t = t0 + 16 * i + r16;
+    if (t >= T) continue;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      const int n = n0 + 16 * j + 4 * qd;
+      if (n >= N) continue;
+      float f[8] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3], 0.f, 0.f, 0.f, 0.f};
+      if (gate) {
+        float g[8];
+        const u32x2 g2 = *(const u32x2*)((const char*)gate + (t * gate_stride + h * N + n) * 2);
+        unpack16<Tag>(u32x4{g2[0], g2[1], 0u, 0u}, g);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) f[e] /= 1.f + expf(-g[e]);
+      }
+      const u32x4 pk = pack16<Tag>(f);
+      *(u32x2*)((char*)out + (t * out_stride + h * out_head + n) * 2) = u32x2{pk[0], pk[1]};
+    }
+  }
+}
+
+// any type, size and alignment: one workgroup per (token, head), the token's row in LDS, a thread per output
+template <typename Tag>
+__global__ void __launch_bounds__(kBlock)
+head_linear_kernel(void* out, int64_t out_stride, int64_t out_head, const void* x, int64_t x_stride, int64_t x_head,
+                   const void* w, const void* gate, int64_t gate_stride, int N, int K) {
+  typedef Elem<Tag> E;
+  extern __shared__ float smem[];
+  const int64_t t = blockIdx.x, h = blockIdx.y;
+  for (int k = threadIdx.x; k < K; k += blockDim.x) smem[k] = E::load(x, t * x_stride + h * x_head + k);
+  __syncthreads();
+  for (int n = threadIdx.x; n < N; n += blockDim.x) {
+    const int64_t row = (h * N + n) * (int64_t)K;
+    float acc = 0.f;
+    for (int k = 0; k < K; ++k) acc += smem[k] * E::load(w, row + k);
+    if (gate) acc /= 1.f + expf(-E::load(gate, t * gate_stride + h * N + n));
+    E::store(out, t * out_stride + h * out_head + n, acc);
   }
 }
 
@@ -148,37 +627,92 @@ extern "C" int sp_rotary_interleaved(void* x, const int64_t* positions, const fl
 }
 
 extern "C" int sp_latent_kv_store(void* pool, int64_t pool_stride, const void* dkv, int64_t dkv_stride,
-                                  const float* norm_w, const int64_t* positions, const float* freq, float mag,
-                                  const int64_t* loc, int64_t num_tokens, int rank, int rot_dim, int rot_dims, float eps,
-                                  int dtype, void* stream) {
+                                  const float* norm_w, void* q, int64_t q_stride, int64_t q_head_stride, int q_offset,
+                                  int heads, const int64_t* positions, const float* freq, float mag, const int64_t* loc,
+                                  int64_t num_tokens, int rank, int rot_dim, int rot_dims, float eps, int dtype, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && rank > 0 && rot_dim >= 0 && rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0);
   if (num_tokens == 0) return SP_OK;
-  SP_CHECK_ARG(pool && dkv && norm_w && positions && loc && (freq || rot_dims == 0));
-  SP_CHECK_ARG(pool_stride >= rank + rot_dim && dkv_stride >= rank + rot_dim);
+  SP_CHECK_ARG((pool || q) && positions && (freq || rot_dims == 0));
+  SP_CHECK_ARG(!pool || (dkv && norm_w && loc && pool_stride >= rank + rot_dim && dkv_stride >= rank + rot_dim));
+  SP_CHECK_ARG(!q || (heads > 0 && q_offset >= 0 && q_head_stride >= q_offset + rot_dims));
+  if (rot_dims > kMaxRot) return SP_ERR_UNSUPPORTED;
   SP_DISPATCH_DTYPE(dtype, (latent_kv_store_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(
-                               pool, pool_stride, dkv, dkv_stride, norm_w, positions, freq, mag, loc, rank, rot_dim, rot_dims, eps)));
+                               pool, pool_stride, dkv, dkv_stride, norm_w, q, q_stride, q_head_stride, q_offset, heads, positions,
+                               freq, mag, loc, rank, rot_dim, rot_dims, eps)));
   SP_LAUNCH_CHECK();
   return SP_OK;
 }
 
-extern "C" int sp_latent_attention(void* out, const void* q_lat, const void* q_rot, const void* pool, int64_t pool_stride,
-                                   const int32_t* req_to_token, int64_t table_stride, int64_t num_tokens, int heads,
-                                   int rank, int rot_dim, int64_t qrot_token_stride, int64_t qrot_head_stride,
-                                   float scale, SP_SEQ_PARAMS, int dtype, void* stream) {
+extern "C" int sp_latent_attention(void* out, const void* q_lat, int64_t lat_token_stride, int64_t lat_head_stride,
+                                   const void* q_rot, const void* pool, int64_t pool_stride, const int32_t* req_to_token,
+                                   int64_t table_stride, int64_t num_tokens, int heads, int rank, int rot_dim,
+                                   int64_t qrot_token_stride, int64_t qrot_head_stride, float scale, int matrix, int splits,
+                                   float* workspace, int64_t workspace_floats, SP_SEQ_PARAMS, int dtype, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && heads > 0 && rank > 0 && rot_dim >= 0);
   if (num_tokens == 0) return SP_OK;
   SP_CHECK_ARG(out && q_lat && pool && req_to_token && req_pool_indices && seq_lens && (q_rot || rot_dim == 0));
   SP_CHECK_ARG(!extend_seq_lens || (extend_prefix_lens && extend_start_loc && token_req));
   SP_CHECK_ARG(extend_seq_lens || num_tokens == batch_size);
-  SP_CHECK_ARG(pool_stride >= rank + rot_dim);
+  SP_CHECK_ARG(pool_stride >= rank + rot_dim && lat_token_stride >= rank && lat_head_stride >= rank);
+  SEQ_BATCH(s);
+  // 16-bit rows of whole 16-byte pieces, widths the tile shapes cover: the matrix cores; anything else: the vector kernel
+  const bool al16 = (((uintptr_t)q_lat | (uintptr_t)q_rot | (uintptr_t)pool | (uintptr_t)workspace) & 15) == 0 &&
+                    ((uintptr_t)out & 7) == 0;
+  if (matrix && (dtype == SP_BF16 || dtype == SP_F16) && rank % 8 == 0 && rot_dim % 8 == 0 && rank <= 512 &&
+      rank + rot_dim <= 576 && al16 && lat_token_stride % 8 == 0 && lat_head_stride % 8 == 0 && qrot_token_stride % 8 == 0 &&
+      qrot_head_stride % 8 == 0 && pool_stride % 8 == 0) {
+    if (splits < 1) splits = 1;
+    SP_CHECK_ARG(splits == 1 || (workspace && splits <= 65535));
+    if (splits > 1 && workspace_floats < (int64_t)splits * num_tokens * heads * (rank + 2)) return SP_ERR_WORKSPACE;
+    const LatentArgs a{out, q_lat, q_rot, pool, req_to_token, workspace, lat_token_stride, lat_head_stride, qrot_token_stride,
+                       qrot_head_stride, pool_stride, table_stride, num_tokens, heads, rank, rot_dim, splits, scale};
+    return dtype == SP_BF16 ? launch_latent<bf16_tag>(a, s, (hipStream_t)stream)
+                            : launch_latent<f16_tag>(a, s, (hipStream_t)stream);
+  }
   if (rank > 64 * kMaxPerLane) return SP_ERR_UNSUPPORTED;
   const size_t lds = 4 * (size_t)(rank + rot_dim + 64) * sizeof(float);
   if (lds > 64 * 1024) return SP_ERR_UNSUPPORTED;
-  SEQ_BATCH(s);
   const dim3 grid((unsigned)num_tokens, (unsigned)((heads + 3) / 4));
   SP_DISPATCH_DTYPE(dtype, (latent_attention_kernel<Tag><<<grid, 256, lds, (hipStream_t)stream>>>(
-                               out, q_lat, q_rot, pool, pool_stride, req_to_token, table_stride, s, num_tokens, heads,
-                               rank, rot_dim, qrot_token_stride, qrot_head_stride, scale)));
+                               out, q_lat, lat_token_stride, lat_head_stride, q_rot, pool, pool_stride, req_to_token, table_stride,
+                               s, num_tokens, heads, rank, rot_dim, qrot_token_stride, qrot_head_stride, scale)));
+  SP_LAUNCH_CHECK();
+  return SP_OK;
+}
+
+extern "C" int sp_head_linear(void* out, int64_t out_stride, int64_t out_head_stride, const void* x, int64_t x_stride,
+                              int64_t x_head_stride, const void* w, const void* gate, int64_t gate_stride,
+                              int64_t num_tokens, int heads, int n, int k, int dtype, void* stream) {
+  SP_CHECK_ARG(num_tokens >= 0 && heads > 0 && n > 0 && k > 0);
+  if (num_tokens == 0) return SP_OK;
+  SP_CHECK_ARG(out && x && w && x_head_stride >= k && out_head_stride >= n && heads <= 65535);
+  SP_CHECK_ARG(x_stride >= (heads - 1) * x_head_stride + k && out_stride >= (heads - 1) * out_head_stride + n);
+  SP_CHECK_ARG(!gate || gate_stride >= (int64_t)heads * n);
+  const bool al = (((uintptr_t)x | (uintptr_t)w) & 15) == 0 && (((uintptr_t)out | (uintptr_t)gate) & 7) == 0 &&
+                  x_stride % 8 == 0 && x_head_stride % 8 == 0 && k % 8 == 0 && n % 4 == 0 && out_stride % 4 == 0 &&
+                  out_head_stride % 4 == 0 && (!gate || gate_stride % 4 == 0);
+  hipStream_t st = (hipStream_t)stream;
+  if (al && (dtype == SP_BF16 || dtype == SP_F16)) {
+#define SP_HL(Tag, TT, NT, TW)                                                                                          \
+  head_linear_mfma_kernel<Tag, TT, NT, TW><<<dim3((unsigned)((num_tokens + 16 * TT * TW - 1) / (16 * TT * TW)),            \
+                                                  (unsigned)((n + 16 * NT * (4 / TW) - 1) / (16 * NT * (4 / TW))),        \
+                                                  (unsigned)heads), 256, 0, st>>>(                                        \
+      out, out_stride, out_head_stride, x, x_stride, x_head_stride, w, gate, gate_stride, num_tokens, n, k)
+    if (num_tokens <= 64) {
+      if (dtype == SP_BF16) SP_HL(bf16_tag, 1, 1, 1);
+      else SP_HL(f16_tag, 1, 1, 1);
+    } else {
+      if (dtype == SP_BF16) SP_HL(bf16_tag, 2, 4, 4);
+      else SP_HL(f16_tag, 2, 4, 4);
+    }
+#undef SP_HL
+    SP_LAUNCH_CHECK();
+    return SP_OK;
+  }
+  const size_t lds = (size_t)k * sizeof(float);
+  if (lds > 64 * 1024) return SP_ERR_UNSUPPORTED;
+  SP_DISPATCH_DTYPE(dtype, (head_linear_kernel<Tag><<<dim3((unsigned)num_tokens, (unsigned)heads), kBlock, lds, st>>>(
+                               out, out_stride, out_head_stride, x, x_stride, x_head_stride, w, gate, gate_stride, n, k)));
   SP_LAUNCH_CHECK();
   return SP_OK;
 }

@@ -146,6 +146,11 @@ __device__ __forceinline__ u32x4 pack16<f16_tag>(const float* f) {
 // fused prologue of sp_gemm_skinny, which must agree bit for bit)
 __device__ __forceinline__ float silu_ref(float a) { return __fdiv_rn(a, __fadd_rn(1.0f, expf(-a))); }
 
+// the tanh form of GELU in fp32 (sp_gelu_tanh_and_mul and the fused epilogue of sp_gemm_skinny share it)
+__device__ __forceinline__ float gelu_tanh_f32(float a) {
+  return 0.5f * a * (1.0f + tanhf(0.7978845608028654f * (a + 0.044715f * a * a * a)));
+}
+
 __device__ __forceinline__ u32x4 ld16(const void* p) { return *(const u32x4*)p; }
 __device__ __forceinline__ void st16(void* p, const u32x4& v) { *(u32x4*)p = v; }
 
@@ -198,7 +203,7 @@ __device__ __forceinline__ float wave_sum(float v) {
   return v;
 }
 
-// sum over N neighbouring lanes (aligned groups of N = 1, 2, 4 or 8) by data-parallel-primitive moves - register-to-register,
+// sum over N neighbouring lanes (aligned groups of N = 1, 2, 4, 8 or 16) by data-parallel-primitive moves - register-to-register,
 // no trip through the LDS crossbar that __shfl_xor takes; every lane of a group ends with the same value
 template <int CTRL>
 __device__ __forceinline__ float dpp_f32(float v) {
@@ -206,10 +211,11 @@ __device__ __forceinline__ float dpp_f32(float v) {
 }
 template <int N>
 __device__ __forceinline__ float lanes_sum(float v) {
-  static_assert(N == 1 || N == 2 || N == 4 || N == 8, "lanes per group");
+  static_assert(N == 1 || N == 2 || N == 4 || N == 8 || N == 16, "lanes per group");
   if constexpr (N >= 2) v += dpp_f32<0xB1>(v);      // quad_perm [1,0,3,2]: lane ^ 1
   if constexpr (N >= 4) v += dpp_f32<0x4E>(v);      // quad_perm [2,3,0,1]: lane ^ 2
   if constexpr (N >= 8) v += dpp_f32<0x141>(v);     // row_half_mirror: lane i <-> 7 - i of each 8 (the other quad's sum)
+  if constexpr (N >= 16) v += dpp_f32<0x140>(v);    // row_mirror: lane i <-> 15 - i of each 16 (the other eight's sum)
   return v;
 }
 

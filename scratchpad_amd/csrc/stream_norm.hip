@@ -1,5 +1,5 @@
 // fp32 residual stream of parallel-sublayer models:  x <- x + mixer(shift(h)) + ff(h),  h = x / rms(x) * w.
-//   scaled embedding      x[t]  = embed[id[t]] * scale                                     (fp32)
+//   scaled embedding      x[t]  = embed[id[t]] * scale (+ table[position[t]])              (fp32)
 //   norm + token shift    h[t]  = x[t] / sqrt(mean(x[t]^2) + eps) * w                      (what the feed-forward reads)
 //                         hs[t] = h[t] + (h[t-1] - h[t]) * mu                              (what the mixer reads)
 //                         h[-1] of a step's first row = the request's saved h (zeros at a sequence's first token)
@@ -14,7 +14,8 @@
 //                         `groups` equal consecutive parts of the row divided by its own root mean square
 // and of post-norm models, whose stream is normed after every sum:
 //   scaled sum + norm     x = N(alpha x + scale * y) w, y a sublayer's result or, in the same pass, a mixture's experts
-//                         weighted and added (an expert may be the row itself) beside a gated dense branch
+//                         weighted and added (an expert may be the row itself) beside a gated dense branch, or two
+//                         branches (N(a) wa + N(b) wb) / 2
 // All arithmetic is fp32; h and hs are rounded once, to the projections' element type.
 #include "seq_batch.h"
 
@@ -23,13 +24,17 @@ namespace {
 
 template <typename Tag>
 __global__ void embed_scale_kernel(float* x, int64_t x_stride, void* lo, int64_t lo_stride, const void* embed,
-                                   const int64_t* ids, int width, int64_t vocab, float scale) {
+                                   const int64_t* ids, const void* table, const int64_t* positions, int64_t table_rows,
+                                   int width, int64_t vocab, float scale) {
   typedef Elem<Tag> E;
   const int64_t t = blockIdx.x;
   int64_t id = ids[t];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  int64_t p = table ? positions[t] : 0;
+  p = p < 0 ? 0 : (p >= table_rows ? table_rows - 1 : p);
   for (int i = threadIdx.x; i < width; i += blockDim.x) {
-    const float v = E::load(embed, id * width + i) * scale;
+    float v = E::load(embed, id * width + i) * scale;
+    if (table) v += E::load(table, p * width + i);
     x[t * x_stride + i] = v;
     if (lo) E::store(lo, t * lo_stride + i, v);
   }
@@ -469,7 +474,7 @@ add_group_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_s
 }
 
 // ---- x = N(alpha x + scale * y) weight in place (+ the new x in the projections' type) -------------------------------
-// y = a, or the mixture's result assembled here: sum over k < top, in that order, of weights[t, k] times the row
+// y = a, or (N(a) wa + N(b) wb) / 2 with a second branch, or the mixture's result assembled here: sum over k < top, in that order, of weights[t, k] times the row
 // z[place[t * top + k]] - or times x itself for an id from `experts` on - and then, with a dense branch, gate[t] * a.
 struct MixRows {
   const void* z;               // null: no mixture
@@ -479,12 +484,17 @@ struct MixRows {
   const float* gate;           // factor of a's row (null: 1)
   int experts, top;
 };
+struct Branch {                // a second result beside a, each normed over the row with its weight
+  const void* b;               // null: none
+  int64_t stride;
+  const float *wa, *wb;
+};
 
 // rows of NV x 256 vectors of 16 bytes at most: a thread holds its part of the row in registers
 template <typename Tag, int NV>
 __global__ void __launch_bounds__(kBlock)
-post_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, MixRows mix, const float* scale, float alpha,
-                     const float* weight, void* lo, int64_t lo_stride, int width, float eps) {
+post_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, Branch br, MixRows mix, const float* scale,
+                     float alpha, const float* weight, void* lo, int64_t lo_stride, int width, float eps) {
   typedef Elem<Tag> E;
   constexpr int V = E::kVec;
   __shared__ float red[kBlock / 64];
@@ -502,6 +512,51 @@ post_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride
       if (a) unpack16<Tag>(ld16((const char*)a + (t * a_stride + c) * E::kBytes), y[u]);
 #pragma unroll
       for (int q = 0; q < V / 4; ++q) unpack16<f32_tag>(ld16(x + t * x_stride + c + 4 * q), xs[u] + 4 * q);
+    }
+  }
+  if (br.b) {
+    __shared__ float red2[2 * (kBlock / 64)];
+    float yb[NV][V], sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int vi = threadIdx.x + u * kBlock;
+#pragma unroll
+      for (int e = 0; e < V; ++e) yb[u][e] = 0.f;
+      if (vi < nvec) unpack16<Tag>(ld16((const char*)br.b + (t * br.stride + (int64_t)vi * V) * E::kBytes), yb[u]);
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        sa += y[u][e] * y[u][e];
+        sb += yb[u][e] * yb[u][e];
+      }
+    }
+    sa = wave_sum(sa);
+    sb = wave_sum(sb);
+    const int wave = threadIdx.x >> 6;
+    if ((threadIdx.x & 63) == 0) {
+      red2[2 * wave] = sa;
+      red2[2 * wave + 1] = sb;
+    }
+    __syncthreads();
+    sa = sb = 0.f;
+    for (int w = 0; w < kBlock / 64; ++w) {
+      sa += red2[2 * w];
+      sb += red2[2 * w + 1];
+    }
+    const float ia = 0.5f / sqrtf(sa / (float)width + eps), ib = 0.5f / sqrtf(sb / (float)width + eps);
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int vi = threadIdx.x + u * kBlock;
+      if (vi < nvec) {
+#pragma unroll
+        for (int q = 0; q < V / 4; ++q) {
+          float fa[4], fb[4];
+          unpack16<f32_tag>(ld16(br.wa + (int64_t)vi * V + 4 * q), fa);
+          unpack16<f32_tag>(ld16(br.wb + (int64_t)vi * V + 4 * q), fb);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            y[u][4 * q + e] = y[u][4 * q + e] * ia * fa[e] + yb[u][4 * q + e] * ib * fb[e];
+        }
+      }
     }
   }
   if (mix.z) {
@@ -575,17 +630,30 @@ post_norm_vec_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride
 // any width and alignment; the row's sum waits in LDS (a thread reads back only what it wrote)
 template <typename Tag>
 __global__ void __launch_bounds__(kBlock)
-post_norm_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, MixRows mix, const float* scale, float alpha,
-                 const float* weight, void* lo, int64_t lo_stride, int width, float eps) {
+post_norm_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, Branch br, MixRows mix, const float* scale,
+                 float alpha, const float* weight, void* lo, int64_t lo_stride, int width, float eps) {
   typedef Elem<Tag> E;
   extern __shared__ float rowbuf[];
   __shared__ float red[kBlock / 64];
   const int64_t t = blockIdx.x;
   const float ga = (a && mix.gate) ? mix.gate[t] : 1.f;
-  float ss = 0.f;
+  float ss = 0.f, ia = 1.f, ib = 0.f;
+  if (br.b) {
+    float sa = 0.f, sb = 0.f;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+      const float u = E::load(a, t * a_stride + i), v = E::load(br.b, t * br.stride + i);
+      sa += u * u;
+      sb += v * v;
+    }
+    sa = block_sum(sa, red);
+    sb = block_sum(sb, red);
+    ia = 0.5f / sqrtf(sa / (float)width + eps);
+    ib = 0.5f / sqrtf(sb / (float)width + eps);
+  }
   for (int i = threadIdx.x; i < width; i += blockDim.x) {
     const float xv = x[t * x_stride + i];
     float y = a ? E::load(a, t * a_stride + i) : 0.f;
+    if (br.b) y = y * ia * br.wa[i] + E::load(br.b, t * br.stride + i) * ib * br.wb[i];
     if (mix.z) {
       float m = 0.f, self = 0.f;
       for (int k = 0; k < mix.top; ++k) {
@@ -612,7 +680,8 @@ post_norm_kernel(float* x, int64_t x_stride, const void* a, int64_t a_stride, Mi
 
 using namespace sp;
 
-extern "C" int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a_stride, const void* z, const int32_t* ids,
+extern "C" int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a_stride, const void* b, int64_t b_stride,
+                            const float* wa, const float* wb, const void* z, const int32_t* ids,
                             const int32_t* place, const float* weights, const float* gate, int experts, int top,
                             const float* scale, float alpha, const float* weight, void* lo, int64_t lo_stride,
                             int64_t num_tokens, int width, float eps, int dtype, void* stream) {
@@ -620,6 +689,8 @@ extern "C" int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a
   if (num_tokens == 0) return SP_OK;
   SP_CHECK_ARG(x && weight && x_stride >= width && (a || z) && (!a || a_stride >= width) && (!lo || lo_stride >= width));
   SP_CHECK_ARG(z ? (ids && place && weights && experts > 0 && top > 0) : !gate);
+  SP_CHECK_ARG(!b || (a && !z && wa && wb && b_stride >= width));
+  const sp::Branch br{b, b_stride, wa, wb};
   const sp::MixRows mix{z, ids, place, weights, gate, experts, top};
   // rows of 16-byte vectors that 256 threads hold in registers: the vector kernel; anything else: the scalar one
   const int vecn = dtype == SP_F32 ? 4 : 8, esize = dtype == SP_F32 ? 4 : 2;
@@ -627,11 +698,12 @@ extern "C" int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a
     return !p || ((((uintptr_t)p) & 15) == 0 && (stride * elem_bytes) % 16 == 0);
   };
   if (width % vecn == 0 && width / vecn <= 4 * kBlock && al(x, x_stride, 4) && al(a, a_stride, esize) && al(z, 0, esize) &&
+      al(b, b_stride, esize) && al(wa, 0, 4) && al(wb, 0, 4) &&
       al(lo, lo_stride, esize) && al(weight, 0, 4) && al(scale, 0, 4)) {
     const int nv = (width / vecn + kBlock - 1) / kBlock;
 #define SP_PN(NV)                                                                                                       \
   SP_DISPATCH_DTYPE(dtype, (post_norm_vec_kernel<Tag, NV><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(  \
-                               x, x_stride, a, a_stride, mix, scale, alpha, weight, lo, lo_stride, width, eps)))
+                               x, x_stride, a, a_stride, br, mix, scale, alpha, weight, lo, lo_stride, width, eps)))
     if (nv <= 1) SP_PN(1);
     else if (nv <= 2) SP_PN(2);
     else SP_PN(4);
@@ -641,18 +713,20 @@ extern "C" int sp_post_norm(float* x, int64_t x_stride, const void* a, int64_t a
   }
   SP_DISPATCH_DTYPE(dtype, (post_norm_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, (size_t)width * sizeof(float),
                                                      (hipStream_t)stream>>>(
-                               x, x_stride, a, a_stride, mix, scale, alpha, weight, lo, lo_stride, width, eps)));
+                               x, x_stride, a, a_stride, br, mix, scale, alpha, weight, lo, lo_stride, width, eps)));
   SP_LAUNCH_CHECK();
   return SP_OK;
 }
 
 extern "C" int sp_embed_scale(float* x, int64_t x_stride, void* lo, int64_t lo_stride, const void* embed, const int64_t* ids,
-                              int64_t num_tokens, int width, int64_t vocab, float scale, int dtype, void* stream) {
+                              const void* table, const int64_t* positions, int64_t table_rows, int64_t num_tokens, int width,
+                              int64_t vocab, float scale, int dtype, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && width > 0 && vocab > 0);
   if (num_tokens == 0) return SP_OK;
   SP_CHECK_ARG(x && embed && ids && x_stride >= width && (!lo || lo_stride >= width));
+  SP_CHECK_ARG(!table || (positions && table_rows > 0));
   SP_DISPATCH_DTYPE(dtype, (embed_scale_kernel<Tag><<<dim3((unsigned)num_tokens), kBlock, 0, (hipStream_t)stream>>>(
-                               x, x_stride, lo, lo_stride, embed, ids, width, vocab, scale)));
+                               x, x_stride, lo, lo_stride, embed, ids, table, positions, table_rows, width, vocab, scale)));
   SP_LAUNCH_CHECK();
   return SP_OK;
 }

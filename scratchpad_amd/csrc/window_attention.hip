@@ -4,7 +4,8 @@
 // lies wholly before the window (block b = positions bP .. bP + P - 1, seen once bP + P - 1 <= p - size), ONE key and
 // value: the means of the block's cached keys and values.  Tokens and blocks share one softmax.  Tokens that left the
 // window while their block is still incomplete behind it are not seen.  size <= 0 means no window (plain causal),
-// P <= 0 no pooling.
+// P <= 0 no pooling.  With `keep_first` = n > 0 (and no pooling) the tokens j < n stay visible to every later query: they are
+// numbered like blocks of one token whose mean is the token itself, of which only the first n exist.
 //
 // Cache: per token a key row [G, D] (rotated) and a value row [G, Dv] (each head divided by its root mean square); the
 // pooled key/value of block b lives in a second pair of buffers at the slot of the block's LAST token, written by the
@@ -312,8 +313,8 @@ __global__ void __launch_bounds__(1024)
 window_attention_kernel(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kpool, const void* vpool,
                         const void* kpooled, const void* vpooled, int64_t kp_stride, int64_t vp_stride,
                         const int32_t* req_to_token, int64_t table_stride, SeqBatch s, int H, int G, int D, int Dv,
-                        int64_t size, int P, float scale, const float* sinks, float softcap, const float* head_bias,
-                        const void* gate, int64_t gate_stride) {
+                        int64_t size, int P, int64_t lead, float scale, const float* sinks, float softcap,
+                        const float* head_bias, const void* gate, int64_t gate_stride) {
   typedef Elem<Tag> E;
   extern __shared__ float smem[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, NW = blockDim.x >> 6;
@@ -328,7 +329,8 @@ window_attention_kernel(void* out, int64_t out_stride, const void* q, int64_t q_
   seq_of_token(s, t, b, start, prefix);
   const int64_t pos = prefix + (t - start);
   const int64_t w0 = (size > 0 && pos - size + 1 > 0) ? pos - size + 1 : 0;      // first token of the window
-  const int64_t nb = (size > 0 && P > 0) ? w0 / P : 0;                            // blocks wholly before it
+  int64_t nb = (size > 0 && P > 0) ? w0 / P : 0;                                  // blocks wholly before it
+  if (nb > lead) nb = lead;                                                       // (no more of them exist)
   const int64_t total = nb + (pos - w0 + 1);
   const int g = h / (H / G);
   const int32_t* table = req_to_token + load_idx(s.req_pool_indices, b, s.idx64) * table_stride;
@@ -474,7 +476,7 @@ __global__ void __launch_bounds__(256)
 window_attention_mfma_kernel(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kpool,
                              const void* vpool, const void* kpooled, const void* vpooled, int64_t kp_stride, int64_t vp_stride,
                              const int32_t* req_to_token, int64_t table_stride, SeqBatch s, int H, int G, int64_t size, int P,
-                             float scale, const float* sinks, float softcap, const float* head_bias, const void* gate,
+                             int64_t lead, float scale, const float* sinks, float softcap, const float* head_bias, const void* gate,
                              int64_t gate_stride) {
   constexpr int D = 32 * DS, Dv = 16 * DT;
   __shared__ uint16_t vt[Dv][kVtRow];
@@ -496,13 +498,15 @@ window_attention_mfma_kernel(void* out, int64_t out_stride, const void* q, int64
   const bool pooled = size > 0 && P > 0;
   const int64_t w0U = (size > 0 && pos0 - size + 1 > 0) ? pos0 - size + 1 : 0;
   const int64_t w0L = (size > 0 && pos_last - size + 1 > 0) ? pos_last - size + 1 : 0;
-  const int64_t nbU = pooled ? w0L / P : 0;
+  int64_t nbU = pooled ? w0L / P : 0;
+  if (nbU > lead) nbU = lead;
   const int64_t totalU = nbU + (pos_last - w0U + 1);
   // this lane's query (column r16 of every S^T tile)
   const bool qvalid = r16 < rows;
   const int64_t pos_q = pos0 + r16;
   const int64_t w0_q = (size > 0 && pos_q - size + 1 > 0) ? pos_q - size + 1 : 0;
-  const int64_t nb_q = pooled ? w0_q / P : 0;
+  int64_t nb_q = pooled ? w0_q / P : 0;
+  if (nb_q > lead) nb_q = lead;
   for (int h0 = 0; h0 < R; h0 += 4) {
     const int hq = g * R + h0 + wave;
     const bool work = h0 + wave < R;
@@ -716,13 +720,21 @@ extern "C" int sp_window_attention(void* out, int64_t out_stride, const void* q,
                                    const void* vpool, const void* kpooled, const void* vpooled, int64_t kp_stride,
                                    int64_t vp_stride, const int32_t* req_to_token, int64_t table_stride,
                                    int64_t num_tokens, int heads, int kv_heads, int dim, int vdim, int64_t window, int block,
-                                   float scale, const float* sinks, float softcap, int sigmoid_weights,
+                                   int keep_first, float scale, const float* sinks, float softcap, int sigmoid_weights,
                                    const float* head_bias, const void* gate, int64_t gate_stride, int matrix, SP_SEQ_PARAMS,
                                    int dtype, void* stream) {
   SP_CHECK_ARG(num_tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0);
   if (num_tokens == 0) return SP_OK;
   SP_CHECK_ARG(out && q && kpool && vpool && req_to_token && req_pool_indices && seq_lens);
   SP_CHECK_ARG((kpooled && vpooled) || block <= 0 || window <= 0);
+  SP_CHECK_ARG(keep_first >= 0 && (keep_first == 0 || block <= 0));
+  int64_t lead = INT64_MAX;                      // how many blocks exist at most
+  if (keep_first > 0) {                          // the kept tokens: blocks of one token, read from the token rows
+    block = 1;
+    lead = keep_first;
+    kpooled = kpool;
+    vpooled = vpool;
+  }
   SP_CHECK_ARG(!extend_seq_lens || (extend_prefix_lens && extend_start_loc && token_req));
   SP_CHECK_ARG(extend_seq_lens || num_tokens == batch_size);
   SP_CHECK_ARG(q_stride >= (int64_t)heads * dim && out_stride >= (int64_t)heads * vdim);
@@ -744,7 +756,7 @@ extern "C" int sp_window_attention(void* out, int64_t out_stride, const void* q,
 #define SP_WM2(T, DS, DT, SG)                                                                                            \
   window_attention_mfma_kernel<T, DS, DT, SG><<<mgrid, 256, 0, (hipStream_t)stream>>>(                                     \
       out, out_stride, q, q_stride, kpool, vpool, kpooled, vpooled, kp_stride, vp_stride, req_to_token, table_stride, s, heads, \
-      kv_heads, window, block, scale, sinks, softcap, head_bias, gate, gate_stride)
+      kv_heads, window, block, lead, scale, sinks, softcap, head_bias, gate, gate_stride)
 #define SP_WM(T, DS, DT)                    \
   do {                                      \
     if (sigmoid_weights) SP_WM2(T, DS, DT, true); \
@@ -772,7 +784,7 @@ extern "C" int sp_window_attention(void* out, int64_t out_stride, const void* q,
 #define SP_WA(V, SG)                                                                                                   \
   SP_DISPATCH_DTYPE(dtype, (window_attention_kernel<Tag, V, SG><<<grid, 64 * nw, lds, (hipStream_t)stream>>>(           \
                                out, out_stride, q, q_stride, kpool, vpool, kpooled, vpooled, kp_stride, vp_stride,      \
-                               req_to_token, table_stride, s, heads, kv_heads, dim, vdim, window, block, scale, sinks,  \
+                               req_to_token, table_stride, s, heads, kv_heads, dim, vdim, window, block, lead, scale, sinks, \
                                softcap, head_bias, gate, gate_stride)))
   if (vec && sigmoid_weights) SP_WA(true, true);
   else if (vec) SP_WA(true, false);

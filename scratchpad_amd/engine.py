@@ -61,6 +61,9 @@ class Engine:
         """parts: (Req, next tokens) per request of the step.  Returns (LogitsProcessorOutput, ScheduleBatch): one
         logits row per request (its last token), or exactly ``logit_rows`` (indices into the step's token rows)."""
         reqs = [r for r, _ in parts]
+        for r, toks in parts:
+            if r.seqlen + len(toks) > self.config.context_len:
+                raise ValueError(f"request {r.rid}: {r.seqlen} + {len(toks)} tokens exceed the context of {self.config.context_len}")
         decode = all(len(t) == 1 and r.seqlen > 0 and r.req_pool_idx is not None for r, t in parts)
         for r, toks in parts:
             r.step_prefix = r.seqlen                       # tokens held before this step
@@ -134,6 +137,8 @@ class Engine:
             req.prompt, req.fed, req.limit = [int(t) for t in p], 0, (sp.max_new_tokens if sp is not None else max_new_tokens)
             if not req.prompt:
                 raise ValueError("empty prompt")
+            if len(req.prompt) + req.limit - 1 > self.config.context_len:      # (the last generated token is not fed)
+                raise ValueError(f"prompt {i}: {len(req.prompt)} + {req.limit} tokens exceed the context of {self.config.context_len}")
             waiting.append(req)
         order = list(waiting)
         running: List[Req] = []

@@ -347,18 +347,20 @@ class ShiftedRMSNorm(nn.Module):
 
 
 class GluFF(nn.Module):
-    """Gated feed-forward with the gate and up projections as ONE product: act = "silu": W_down (silu(g) * u);
-    act = "clamped": g' = min(g, limit), u' = clamp(u, -limit, limit), W_down (g' * sigmoid(alpha g') * (u' + 1))."""
+    """Gated feed-forward with the gate and up projections as ONE product: act = "silu": W_down (silu(g) * u); act =
+    "gelu_tanh": the tanh form of GELU in silu's place (one launch with the product in steps of few tokens); act = "clamped": g' = min(g, limit), u' = clamp(u, -limit, limit), W_down (g' * sigmoid(alpha g') * (u' + 1))."""
 
     def __init__(self, width: int, ff: int, act: str = "silu", limit: float = 0.0, alpha: float = 1.702, dtype=None):
         super().__init__()
-        if act not in ("silu", "clamped"):
+        if act not in ("silu", "gelu_tanh", "clamped"):
             raise ValueError(f"unknown activation {act!r}")
         self.ff, self.act, self.limit, self.alpha = ff, act, limit, alpha
         self.gate_up = nn.Parameter(torch.empty(2 * ff, width, dtype=dtype), requires_grad=False)
         self.down = nn.Parameter(torch.empty(width, ff, dtype=dtype), requires_grad=False)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
+        if self.act == "gelu_tanh":
+            return _native.linear(_native.linear_gelu_mul(h, self.gate_up), self.down)
         gu = _native.linear(h, self.gate_up)
         y = _native.silu_and_mul(gu) if self.act == "silu" else _native.moe_glu(gu.contiguous(), self.limit, self.alpha)
         return _native.linear(y, self.down)
@@ -440,18 +442,25 @@ class PostNorm(nn.Module):
     x <- N(alpha x + scale * y) * weight, N = division by the row's root mean square, scale a learned vector (``layer_scale``)
     or 1.  The stream itself is what the next sublayer reads, so the call returns it in the projections' dtype.  y is a
     tensor, or moe.MixtureRows - a mixture whose weighted sum (and identity experts, and gated dense branch) is formed in the
-    same pass over the row."""
+    same pass over the row - or, with ``branches`` = 2, a pair (a, b), each normed over the row with its own weight and
+    averaged: y = (N(a) wa + N(b) wb) / 2."""
 
-    def __init__(self, width: int, eps: float = 1e-6, alpha: float = 1.0, layer_scale: bool = False) -> None:
+    def __init__(self, width: int, eps: float = 1e-6, alpha: float = 1.0, layer_scale: bool = False, branches: int = 1) -> None:
         super().__init__()
         f32 = dict(dtype=torch.float32)
         self.weight = nn.Parameter(torch.ones(width, **f32), requires_grad=False)
         self.scale = nn.Parameter(torch.ones(width, **f32), requires_grad=False) if layer_scale else None
+        self.branch_weight = nn.Parameter(torch.ones(2, width, **f32), requires_grad=False) if branches == 2 else None
         self.variance_epsilon, self.alpha = eps, alpha
 
     def forward(self, x: torch.Tensor, y, dtype: torch.dtype, want_lo: bool = True) -> Optional[torch.Tensor]:
         mix = {}
-        if not isinstance(y, torch.Tensor):
+        if isinstance(y, tuple) != (self.branch_weight is not None):
+            raise RuntimeError("PostNorm: built for another number of branches")
+        if isinstance(y, tuple):
+            y, b = y
+            mix = dict(b=b, wa=self.branch_weight.data[0], wb=self.branch_weight.data[1])
+        elif not isinstance(y, torch.Tensor):
             mix = dict(z=y.z, ids=y.ids, place=y.place, weights=y.weights, gate=y.gate, experts=y.experts)
             y = y.dense
         return _native.post_norm(x, y, self.weight.data, self.variance_epsilon, self.alpha, dtype,

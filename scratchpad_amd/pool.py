@@ -438,12 +438,16 @@ class WindowKVPool(KVCache):
     """Token-level key/value pool whose layers differ in width and whose key and value widths differ: per layer in
     ``layers`` ({layer id: (kv_heads, dim, vdim, pooled)}) a key buffer [P+1, kv_heads * dim] and a value buffer
     [P+1, kv_heads * vdim]; layers with ``pooled`` also get a second pair of the same shape that holds, at the slot of a
-    block's last token, the mean key and value of the block (attention.PooledWindowAttention).  Same slot ids, allocator
-    and dummy slot 0 as MHATokenToKVPool; layers not named take no memory."""
+    block's last token, the mean key and value of the block (attention.PooledWindowAttention).  ``latent``: {layer id: (rank,
+    rot_dim)} of layers that keep LatentTokenToKVPool's row instead - one buffer [P+1, rank + rot_dim], the value being its first
+    rank columns.  Same slot ids, allocator and dummy slot 0 as MHATokenToKVPool; layers not named take no memory."""
 
-    def __init__(self, size: int, dtype: torch.dtype, layers, device: str):
+    def __init__(self, size: int, dtype: torch.dtype, layers, device: str, latent=None):
         if dtype not in (torch.float32, torch.float16, torch.bfloat16):
             raise NotImplementedError(f"window KV cache dtype {dtype} is not built")
+        self.latent = {int(l): (int(r), int(d)) for l, (r, d) in (latent or {}).items()}
+        if set(self.latent) & {int(l) for l in layers}:
+            raise ValueError("a layer keeps either key/value rows or a latent row")
         self.size, self.page_size, self.dtype, self.store_dtype, self.device = size, 1, dtype, dtype, device
         self.layers = {int(l): (int(g), int(d), int(dv), bool(p)) for l, (g, d, dv, p) in layers.items()}
         z = lambda n: torch.zeros((size + 1, n), dtype=dtype, device=device)
@@ -451,11 +455,13 @@ class WindowKVPool(KVCache):
         self._v = {l: z(g * dv) for l, (g, d, dv, p) in self.layers.items()}
         self._kp = {l: z(g * d) for l, (g, d, dv, p) in self.layers.items() if p}
         self._vp = {l: z(g * dv) for l, (g, d, dv, p) in self.layers.items() if p}
-        self.layer_num = len(self.layers)
+        for l, (r, d) in self.latent.items():
+            self._k[l] = z(r + d)
+        self.layer_num = len(self._k)
         self.layer_transfer_counter = None
 
     def _all(self):
-        return [b[l] for l in sorted(self.layers) for b in (self._k, self._v, self._kp, self._vp) if l in b]
+        return [b[l] for l in sorted(self._k) for b in (self._k, self._v, self._kp, self._vp) if l in b]
 
     def get_kv_size_bytes(self):
         return (sum(b.nbytes for d in (self._k, self._kp) for b in d.values()),
@@ -465,10 +471,10 @@ class WindowKVPool(KVCache):
         return self._k[layer_id]
 
     def get_value_buffer(self, layer_id: int) -> torch.Tensor:
-        return self._v[layer_id]
+        return self._k[layer_id][:, :self.latent[layer_id][0]] if layer_id in self.latent else self._v[layer_id]
 
     def get_kv_buffer(self, layer_id: int):
-        return self._k[layer_id], self._v[layer_id]
+        return self.get_key_buffer(layer_id), self.get_value_buffer(layer_id)
 
     def get_pooled_buffers(self, layer_id: int):
         """(keys, values) of the blocks, or (None, None) for a layer without pooling"""
@@ -477,7 +483,8 @@ class WindowKVPool(KVCache):
     def set_kv_buffer(self, layer, loc: torch.Tensor, cache_k: torch.Tensor, cache_v: torch.Tensor) -> None:
         """rows already rotated / normed (the fused store, _native.qkv_rotary_store, is what the model path runs)"""
         self._k[layer.layer_id][loc] = cache_k.reshape(loc.shape[0], -1).to(self.dtype)
-        self._v[layer.layer_id][loc] = cache_v.reshape(loc.shape[0], -1).to(self.dtype)
+        if layer.layer_id not in self.latent:
+            self._v[layer.layer_id][loc] = cache_v.reshape(loc.shape[0], -1).to(self.dtype)
 
     def get_flat_data(self, indices):
         return [b[indices] for b in self._all()]

@@ -1,7 +1,8 @@
 """Recurrent token mixers over per-request state in the RecurrentStatePool: WKVMixer (RWKV-style time mixing, csrc/wkv.hip),
 Mamba2Mixer (state-space duality form, csrc/ssm.hip), MLSTMMixer (matrix memory with exponential gating, csrc/mlstm.hip),
 GeneralDeltaMixer (generalized delta rule, csrc/delta_rule.hip), HGRN2Mixer (linear attention whose forget gate also
-writes, csrc/hgrn.hip) and GatedDeltaMixer (delta rule with a decay per key channel, csrc/gated_delta.hip).
+writes, csrc/hgrn.hip), GatedDeltaMixer (delta rule with a decay per key channel, csrc/gated_delta.hip) and HeadDeltaMixer
+(delta rule with one decay per head, csrc/head_delta.hip).
 
 WKVMixer:
 
@@ -260,3 +261,53 @@ class GatedDeltaMixer(nn.Module):
 
     def forward(self, h: torch.Tensor, forward_batch: ForwardBatch, state_id: Optional[int] = None) -> torch.Tensor:
         return self.scan(_native.linear(h, self.in_proj), forward_batch, state_id)
+
+
+class HeadDeltaMixer(nn.Module):
+    """Delta rule with one decay per head.  q, k [kv_heads, dim] and v [heads, vdim] are projections of h that pass a causal
+    per-channel convolution of ``taps`` taps (no bias; its latest taps - 1 inputs are request state) and silu; value head h reads
+    query/key head h // (heads / kv_heads).  In fp32, per head:
+        qn = q / sqrt(|q|^2 + 1e-6) dim^(-1/2),   kn = k / sqrt(|k|^2 + 1e-6),   beta = sigmoid(W_b x)
+        g  = exp(-exp(A_log) softplus(W_a x + dt_bias))
+        S <- g S;   u = beta (v - S^T kn);   S <- S + kn u^T;   o = S^T qn   (S [dim, vdim])
+    out = W_o (o / rms_head(o) * norm * silu(W_g h)), norm [vdim] shared by the heads.  The rows [q | k | v | g] of the input
+    projection may be part of a larger product of the caller (``scan`` takes the views); ``forward`` runs the mixer's own.  The
+    gate rows [b | a] are a separate fp32 product (a step size or decay is never rounded to 16 bits) of x - h itself, or the
+    fp32 stream that h is a copy of."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float,
+                 layer_id: Optional[int] = None, own_input: bool = True, dtype=None):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("value heads must be a multiple of query/key heads")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.taps, self.eps = heads, kv_heads, dim, vdim, taps, eps
+        self.layer_id = layer_id
+        self.conv_rows = 2 * kv_heads * dim + heads * vdim
+        self.in_rows = self.conv_rows + heads * vdim
+        f32 = dict(dtype=torch.float32)
+        self.in_proj = nn.Parameter(torch.empty(self.in_rows, width, dtype=dtype), requires_grad=False) if own_input else None
+        self.gates = nn.Parameter(torch.zeros(2 * heads, width, **f32), requires_grad=False)       # [b rows | a rows]
+        self.conv = nn.Parameter(torch.zeros(self.conv_rows, taps, **f32), requires_grad=False)
+        self.dt_bias = nn.Parameter(torch.zeros(heads, **f32), requires_grad=False)
+        self.A_log = nn.Parameter(torch.zeros(heads, **f32), requires_grad=False)
+        self.norm = nn.Parameter(torch.ones(vdim, **f32), requires_grad=False)
+        self.o = nn.Parameter(torch.empty(width, heads * vdim, dtype=dtype), requires_grad=False)
+
+    @staticmethod
+    def state_shapes(heads: int, kv_heads: int, dim: int, vdim: int, taps: int):
+        return {"S": (heads, dim, vdim), "conv": (max(taps - 1, 0), 2 * kv_heads * dim + heads * vdim)}
+
+    def scan(self, a: torch.Tensor, x: torch.Tensor, forward_batch: ForwardBatch, state_id: Optional[int] = None) -> torch.Tensor:
+        """a [T, >= in_rows]: the outputs of the rows [q | k | v | g]; x [T, W]: what the gates read -> the mixer's output [T, W]"""
+        seq, states = forward_batch.attn_backend.seq, forward_batch.state_pool
+        sid = self.layer_id if state_id is None else state_id
+        nk, c = self.kv_heads * self.dim, self.conv_rows
+        pre = _native.small_linear_f32(x, self.gates.data)
+        qkv = _native.causal_conv_silu(a[:, :c], self.conv.data, None, states.state(sid, "conv"), seq)
+        o = _native.head_delta_scan(qkv[:, :nk], qkv[:, nk:2 * nk], qkv[:, 2 * nk:], a[:, c:self.in_rows], pre, self.dt_bias.data,
+                                    self.A_log.data, self.norm.data, states.state(sid, "S"), seq, self.heads, self.kv_heads,
+                                    self.dim, self.vdim, self.eps)
+        return _native.linear(o, self.o)
+
+    def forward(self, h: torch.Tensor, forward_batch: ForwardBatch, state_id: Optional[int] = None) -> torch.Tensor:
+        return self.scan(_native.linear(h, self.in_proj), h, forward_batch, state_id)

@@ -50,6 +50,11 @@ def _monolix_config(raw: dict, context_len=None, **_kw):
     return MonolixConfig(raw, context_len=context_len or 8192)
 
 
+def _kirenex_config(raw: dict, context_len=None, **_kw):
+    from .kirenex import KirenexConfig
+    return KirenexConfig(raw, context_len=context_len)
+
+
 def _llama_class():
     from .llama import LlamaForCausalLM
     return LlamaForCausalLM
@@ -85,6 +90,11 @@ def _monolix_class():
     return MonolixForCausalLM
 
 
+def _kirenex_class():
+    from .kirenex import KirenexForCausalLM
+    return KirenexForCausalLM
+
+
 # architecture name -> (configuration from config.json's dict, model class); both lazy so that naming a model does not
 # import the others
 MODELS = {
@@ -94,6 +104,7 @@ MODELS = {
     "Toredra": (_toredra_config, _toredra_class),
     "Kikurax": (_kikurax_config, _kikurax_class),
     "Monolix": (_monolix_config, _monolix_class),
+    "Kirenex": (_kirenex_config, _kirenex_class),
 }
 
 
