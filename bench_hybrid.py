@@ -1,7 +1,7 @@
-"""bench.py --mode hybrid / --mode sominex / --mode toredra / --mode kikurax / --mode monolix: prefill and decode throughput of
-the Tizalorn / the Sominex / the Toredra / the Kikurax / the Monolix design at layer sizes of real models (random weights),
+"""bench.py --mode hybrid / sominex / toredra / kikurax / monolix / kirenex: prefill and decode throughput of the Tizalorn / the
+Sominex / the Toredra / the Kikurax / the Monolix / the Kirenex design at layer sizes of real models (random weights),
 beside a Llama of the same width and depth on the same engine path (the Toredra mode also runs Sominex, the Kikurax mode
-Sominex and Toredra, the Monolix mode Kikurax: their nearest relatives), and a per-kernel table: every HIP kernel
+Sominex and Toredra, the Monolix and Kirenex modes Kikurax: their nearest relatives), and a per-kernel table: every HIP kernel
 (and library product) of both models timed inside an eager prefill batch and an eager decode step, with the time its
 algorithmic bytes and flops would take at the chip's peaks (fraction of roofline).
 
@@ -109,6 +109,28 @@ def monolix_config(width: int, layers: int, context_len: int):
     return MonolixConfig(raw, context_len=context_len)
 
 
+def kirenex_config(width: int, layers: int, context_len: int):
+    """layers in the order latent attention, parallel, latent attention on the first layer's rows, parallel, each with a gated
+    feed-forward: latent rank 512 with 64 rotated dimensions, heads of 128; windowed attention of 128-wide heads with a quarter as
+    many key/value heads, rotation on half of each head, a window of 256 behind which 4 tokens stay; beside it a head-gated delta
+    rule of width / 128 heads with 128 x 128 states over width / 256 query/key heads (4 taps)"""
+    from scratchpad_amd.kirenex import KirenexConfig
+    lat = {"heads": width // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+           "rot": {"base": 50000.0, "dims": 64}}
+    par = {"left": {"heads": width // 128, "kv_heads": max(1, width // 512), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                    "mask": {"size": 256, "keep_first": 4},
+                    "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 4096}}},
+           "right": {"heads": width // 128, "kv_heads": max(1, width // 256), "dim": 128, "vdim": 128, "conv": 4}}
+    dense = {"kind": "dense", "ff": {2048: 8192, 4096: 14336}.get(width, 3 * width)}
+    spec = []
+    for i in range(layers):
+        m = par if i % 2 else ({**lat, "kv_from": i - 2} if i % 4 == 2 else lat)
+        spec.append({"type": "parallel" if i % 2 else "latent_attention", "mixer": m, "mlp": dense})
+    raw = {"architecture": "Kirenex", "vocab": 128256, "width": width, "norm": {"eps": 1e-5}, "postln_alpha": 2.5,
+           "max_positions": max(8192, context_len), "layers": spec}
+    return KirenexConfig(raw, context_len=context_len)
+
+
 def llama_config(width: int, layers: int, context_len: int):
     """the layers of Llama-3.2-1B (width 2048) / Llama-3-8B (width 4096), `layers` of them"""
     from scratchpad_amd.model_runner import ModelConfig
@@ -198,7 +220,7 @@ def instrument(clock: KernelClock, cfg):
 
     def latent(a, k, out):
         q_lat, q_rot, pool = a[0], a[1], a[2]
-        H, T, C = q_lat.shape
+        H, C = q_lat.shape[1 if k.get("token_major") else 0], q_lat.shape[2]
         R = q_rot.shape[2]
         return _nbytes(q_lat, out) + clock.keys_read() * (C + R) * pool.element_size(), 2 * H * clock.pairs() * (2 * C + R), MATRIX
 
@@ -245,6 +267,17 @@ def instrument(clock: KernelClock, cfg):
         q, state, heads, D, Dv = a[0], a[7], a[9], a[11], a[12]
         return _nbytes(*a[:6], out) + 2 * len(clock.step["extend"]) * heads * D * Dv * 4, 6 * q.shape[0] * heads * D * Dv, VECTOR32
 
+    def hdelta(a, k, out):       # one sweep per token: the update (3 flops per state element), the read-out (2), the next S^T k (2)
+        q, state, heads, D, Dv = a[0], a[8], a[10], a[12], a[13]
+        return _nbytes(*a[:5], out) + 2 * len(clock.step["extend"]) * heads * D * Dv * 4, 7 * q.shape[0] * heads * D * Dv, VECTOR32
+
+    def heads(a, k, out):        # a product per head
+        x, w = a[0], a[1]
+        return _nbytes(x, w, k.get("gate"), out), 2 * x.shape[0] * w.numel(), MATRIX
+
+    def glu(a, k, out):          # (no result: the shape is not taken, the caller runs the two steps)
+        return gemm(a, k, out) if out is not None else (0, 0, MATRIX)
+
     def lowrank(a, k, out):
         p, w = a[0], a[1]
         return _nbytes(p, w, out), 2 * p.shape[0] * w.shape[0] * w.shape[1], VECTOR32
@@ -259,12 +292,13 @@ def instrument(clock: KernelClock, cfg):
              "token_shift": io, "wkv_decay": io, "wkv_recurrence": wkv, "rotary_interleaved": io, "latent_kv_store": io,
              "latent_attention": latent, "moe_route": io, "moe_align": io, "moe_grouped_gemm": grouped, "moe_glu": io,
              "moe_combine": io, "rmsnorm": io, "fused_add_rmsnorm": io, "silu_and_mul": io, "rotary_embedding": io,
-             "extend_attention": llama_extend, "decode_attention": llama_extend, "linear": gemm, "linear_silu_mul": gemm,
+             "extend_attention": llama_extend, "decode_attention": llama_extend, "linear": gemm,
              "embed_scale": io, "norm_shift": io, "stream_add": io, "qkv_rotary_store": io, "pool_blocks": io,
              "window_attention": window, "small_linear_f32": small, "causal_conv_silu": io, "mamba2_scan": scan,
              "gated_group_norm": io, "mlstm_scan": mlstm, "moe_route_softmax": io,
              "gated_add_norm": io, "relu_square": io, "scale_softcap": io, "delta_gates": io, "delta_recurrence": delta,
-             "hgrn2_scan": hgrn, "linear_relu_square": gemm, "post_norm": join, "add_group_norm": io, "lowrank_gate": lowrank, "gated_delta_scan": gdelta}
+             "hgrn2_scan": hgrn, "linear_relu_square": gemm, "post_norm": join, "add_group_norm": io, "lowrank_gate": lowrank, "gated_delta_scan": gdelta,
+             "latent_rotate_query": io, "head_linear": heads, "head_delta_scan": hdelta, "gelu_tanh_and_mul": io, "_skinny_glu": glu}
     for name, cost in costs.items():
         saved[name] = getattr(N, name)
         setattr(N, name, clock.record(name, saved[name], cost))
@@ -393,7 +427,7 @@ def hybrid_main(args, design: str = "tizalorn"):
     runs = []
     for w in widths:
         row = {"width": w, "layers": layers}
-        beside = {"toredra": ("sominex", "llama"), "kikurax": ("sominex", "toredra", "llama"), "monolix": ("kikurax", "llama")}.get(design, ("llama",))
+        beside = {"toredra": ("sominex", "llama"), "kikurax": ("sominex", "toredra", "llama"), "monolix": ("kikurax", "llama"), "kirenex": ("kikurax", "llama")}.get(design, ("llama",))
         for model in (design, *beside):
             cmd = [sys.executable, "-u", os.path.abspath(__file__), "--child", model, "--width", str(w), "--layers", str(layers),
                    "--bs", str(args.bs), "--ctx", str(args.ctx), "--steps", str(args.steps), "--warmup", str(args.warmup),
@@ -426,7 +460,7 @@ def child_main():
     import sys
     sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
     ap = argparse.ArgumentParser()
-    ap.add_argument("--child", required=True, choices=["tizalorn", "sominex", "toredra", "kikurax", "monolix", "llama"])
+    ap.add_argument("--child", required=True, choices=["tizalorn", "sominex", "toredra", "kikurax", "monolix", "kirenex", "llama"])
     for name in ("width", "layers", "bs", "ctx", "steps", "warmup", "max-prefill-tokens"):
         ap.add_argument("--" + name, type=int, required=True)
     ap.add_argument("--no-graph", action="store_true")
@@ -436,7 +470,7 @@ def child_main():
         raise SystemExit(DISABLED)
     torch.cuda.set_device(0)
     ctx_len = a.ctx + 2 * (a.steps + a.warmup) + 16
-    cfg = {"sominex": sominex_config, "toredra": toredra_config, "kikurax": kikurax_config, "monolix": monolix_config, "llama": llama_config}[a.child](a.width, a.layers, ctx_len)
+    cfg = {"sominex": sominex_config, "toredra": toredra_config, "kikurax": kikurax_config, "monolix": monolix_config, "kirenex": kirenex_config, "llama": llama_config}[a.child](a.width, a.layers, ctx_len)
     out = run_model(cfg, a, not a.no_kernel_table)
     print("RESULT " + json.dumps(out), flush=True)
 

@@ -1754,7 +1754,7 @@ def gated_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, bpre: to
     return out
 
 
-HEAD_DELTA_WORKGROUPS = 512     # a head's value channels are shared out until a launch has about this many workgroups
+HEAD_DELTA_WORKGROUPS = 256     # a head's value channels are shared out until a launch has about this many workgroups
 
 
 def head_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, pre: torch.Tensor,

@@ -38,31 +38,20 @@ struct HeadDelta {
   float eps;
 };
 
-// element `i` of a row that starts at element `at`, 8 (16-bit) or 4 (fp32) at a time where VEC
-template <typename Tag, bool VEC>
-__device__ __forceinline__ void stage_row(float* dst, const void* src, int64_t at, int i, int n) {
-  typedef Elem<Tag> E;
-  constexpr int V = VEC ? E::kVec : 1;
-  if constexpr (VEC) {
-    float f[V];
-    if (i < n) {
-      unpack16<Tag>(ld16((const char*)src + (at + i) * E::kBytes), f);
-    } else {
-#pragma unroll
-      for (int e = 0; e < V; ++e) f[e] = 0.f;
-    }
-#pragma unroll
-    for (int e = 0; e < V; ++e) dst[i + e] = f[e];
-  } else {
-    dst[i] = i < n ? E::load(src, at + i) : 0.f;
-  }
+// sum over aligned groups of N lanes, N a power of two up to a wave
+template <int N>
+__device__ __forceinline__ float group_sum(float v) {
+  v = lanes_sum<(N < 16 ? N : 16)>(v);
+  if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
+  if constexpr (N >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
 }
 
-template <typename Tag, int KP, bool VEC>
-__global__ void __launch_bounds__(1024)
+template <typename Tag, int KP, bool VEC, int MAXT>
+__global__ void __launch_bounds__(MAXT)
 head_delta_kernel(HeadDelta a, SeqBatch s) {
   typedef Elem<Tag> E;
-  constexpr int kChunk = hd_chunk(KP), SP = hd_lanes(KP), DS = KP / SP, V = VEC ? E::kVec : 1;
+  constexpr int kChunk = hd_chunk(KP), SP = hd_lanes(KP), DS = KP / SP, V = E::kVec;
   static_assert(DS % 4 == 0, "a lane's rows are read four at a time");
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int cols = a.cols, K = a.K, H = a.H, Dv = a.Dv;
@@ -102,38 +91,133 @@ head_delta_kernel(HeadDelta a, SeqBatch s) {
       for (int c = 0; c < kCols; ++c) S[c][ii] = (held && i < K && c0 + c < ncols) ? st[(int64_t)i * Dv + c0 + c] : 0.f;
     }
   }
-  for (int64_t t0 = 0; t0 < len; t0 += kChunk) {
-    const int n = (int)(len - t0 < kChunk ? len - t0 : kChunk);
-    __syncthreads();                                 // the previous pass's epilogue is done with so and sinv
-    for (int e = j; e < n * (KP / V); e += NT) {
-      const int tt = e / (KP / V), i = (e % (KP / V)) * V;
-      const int64_t row = start + t0 + tt;
-      stage_row<Tag, VEC>(sq + tt * KP, a.q, row * a.q_stride + qc, i, K);
-      stage_row<Tag, VEC>(sk + tt * KP, a.k, row * a.k_stride + qc, i, K);
+  // staging in 16-byte pieces: QP pieces (lanes) per row of q and k, vp per row of this workgroup's values
+  constexpr int kAhead = 2, QP = KP / V;
+  const int vp = cols / V;
+  u32x4 fq[kAhead], fk[kAhead], fv[kAhead];
+  float fb = 0.f, fa = 0.f;
+  auto get_qk = [&](int e, int64_t t0, int n, u32x4& rq, u32x4& rk) {
+    const int tt = e / QP, i = (e % QP) * V;
+    const int64_t row = start + t0 + tt;
+    rq = rk = u32x4{0u, 0u, 0u, 0u};
+    if (tt < n && i < K) {
+      rq = ld16((const char*)a.q + (row * a.q_stride + qc + i) * E::kBytes);
+      rk = ld16((const char*)a.k + (row * a.k_stride + qc + i) * E::kBytes);
     }
-    for (int e = j; e < n * (cols / V); e += NT) {
-      const int tt = e / (cols / V), i = (e % (cols / V)) * V;
-      stage_row<Tag, VEC>(sv + tt * cols, a.v, (start + t0 + tt) * a.v_stride + vc, i, ncols);
-    }
+  };
+  auto get_v = [&](int e, int64_t t0, int n, u32x4& rv) {
+    const int tt = e / vp, i = (e % vp) * V;
+    rv = u32x4{0u, 0u, 0u, 0u};
+    if (tt < n && i < ncols) rv = ld16((const char*)a.v + ((start + t0 + tt) * a.v_stride + vc + i) * E::kBytes);
+  };
+  auto get_gates = [&](int64_t t0, int n, float& b_, float& a_) {
     if (j < n) {
       const float* pre = a.pre + (start + t0 + j) * a.pre_stride;
-      sbeta[j] = 1.f / (1.f + expf(-pre[h]));
-      sg[j] = expf(-rate * softplus_hd(pre[H + h] + bias));
+      b_ = pre[h];
+      a_ = pre[H + h];
+    }
+  };
+  auto put_qk = [&](int e, int n, const u32x4& rq, const u32x4& rk) {
+    const int tt = e / QP;
+    if (tt >= n) return;                             // (all lanes of a row or none)
+    float q_[V], k_[V], q2 = 0.f, k2 = 0.f;
+    unpack16<Tag>(rq, q_);
+    unpack16<Tag>(rk, k_);
+#pragma unroll
+    for (int x = 0; x < V; ++x) {
+      q2 += q_[x] * q_[x];
+      k2 += k_[x] * k_[x];
+    }
+    const float iq = qscale * rsqrtf(group_sum<QP>(q2) + 1e-6f), ik = rsqrtf(group_sum<QP>(k2) + 1e-6f);
+#pragma unroll
+    for (int x = 0; x < V; ++x) {
+      q_[x] *= iq;
+      k_[x] *= ik;
+    }
+#pragma unroll
+    for (int x = 0; x < V; x += 4) {
+      st16(sq + e * V + x, pack16<f32_tag>(q_ + x));
+      st16(sk + e * V + x, pack16<f32_tag>(k_ + x));
+    }
+  };
+  auto put_v = [&](int e, int n, const u32x4& rv) {
+    if (e >= n * vp) return;
+    float v_[V];
+    unpack16<Tag>(rv, v_);
+#pragma unroll
+    for (int x = 0; x < V; x += 4) st16(sv + e * V + x, pack16<f32_tag>(v_ + x));
+  };
+  auto put_gates = [&](float b_, float a_) {
+    sbeta[j] = 1.f / (1.f + expf(-b_));
+    sg[j] = expf(-rate * softplus_hd(a_ + bias));
+  };
+  auto fetch = [&](int64_t t0) {
+    const int n = (int)(len - t0 < kChunk ? len - t0 : kChunk);
+#pragma unroll
+    for (int u = 0; u < kAhead; ++u) {
+      get_qk(j + u * NT, t0, n, fq[u], fk[u]);
+      get_v(j + u * NT, t0, n, fv[u]);
+    }
+    get_gates(t0, n, fb, fa);
+  };
+  // which columns of which tokens this thread hands on (several workgroups per head): its column group, every o_step-th token
+  const int og = (ncols + kCols - 1) / kCols, o_step = NT / og, o_col = (j % og) * kCols;
+  const int o_row = j < og * o_step ? j / og : kChunk;
+  if constexpr (VEC) fetch(0);
+  for (int64_t t0 = 0; t0 < len; t0 += kChunk) {
+    const int n = (int)(len - t0 < kChunk ? len - t0 : kChunk);
+    __syncthreads();                                 // the previous pass's readers are done
+    if constexpr (VEC) {
+      // the pieces fetched during the previous pass's token loop, then (small workgroups) what they did not cover: a row's
+      // lanes hold all of it, so its norm is formed on the way
+#pragma unroll
+      for (int u = 0; u < kAhead; ++u) put_qk(j + u * NT, n, fq[u], fk[u]);
+#pragma unroll
+      for (int u = 0; u < kAhead; ++u) put_v(j + u * NT, n, fv[u]);
+      for (int e = j + kAhead * NT; e < n * QP; e += NT) {
+        u32x4 rq, rk;
+        get_qk(e, t0, n, rq, rk);
+        put_qk(e, n, rq, rk);
+      }
+      for (int e = j + kAhead * NT; e < n * vp; e += NT) {
+        u32x4 rv;
+        get_v(e, t0, n, rv);
+        put_v(e, n, rv);
+      }
+      if (j < n) put_gates(fb, fa);
+    } else {
+      for (int e = j; e < n * KP; e += NT) {
+        const int tt = e / KP, i = e % KP;
+        const int64_t row = start + t0 + tt;
+        sq[e] = i < K ? E::load(a.q, row * a.q_stride + qc + i) : 0.f;
+        sk[e] = i < K ? E::load(a.k, row * a.k_stride + qc + i) : 0.f;
+      }
+      for (int e = j; e < n * cols; e += NT) {
+        const int tt = e / cols, i = e % cols;
+        sv[e] = i < ncols ? E::load(a.v, (start + t0 + tt) * a.v_stride + vc + i) : 0.f;
+      }
+      if (j < n) {
+        get_gates(t0, n, fb, fa);
+        put_gates(fb, fa);
+      }
+      __syncthreads();
+      for (int tt = wave; tt < n; tt += waves) {     // unit query and key of every token of the pass: a wave per token
+        float sk2 = 0.f, sq2 = 0.f;
+        for (int i = lane; i < K; i += 64) {
+          sk2 += sk[tt * KP + i] * sk[tt * KP + i];
+          sq2 += sq[tt * KP + i] * sq[tt * KP + i];
+        }
+        const float ik = 1.f / sqrtf(wave_sum(sk2) + 1e-6f), iq = qscale / sqrtf(wave_sum(sq2) + 1e-6f);
+        for (int i = lane; i < K; i += 64) {
+          sk[tt * KP + i] *= ik;
+          sq[tt * KP + i] *= iq;
+        }
+      }
     }
     __syncthreads();
-    for (int tt = wave; tt < n; tt += waves) {       // unit query and key of every token of the pass: a wave per token
-      float sk2 = 0.f, sq2 = 0.f;
-      for (int i = lane; i < K; i += 64) {
-        sk2 += sk[tt * KP + i] * sk[tt * KP + i];
-        sq2 += sq[tt * KP + i] * sq[tt * KP + i];
-      }
-      const float ik = 1.f / sqrtf(wave_sum(sk2) + 1e-6f), iq = qscale / sqrtf(wave_sum(sq2) + 1e-6f);
-      for (int i = lane; i < K; i += 64) {
-        sk[tt * KP + i] *= ik;
-        sq[tt * KP + i] *= iq;
-      }
+    if constexpr (VEC) {
+      if (t0 + kChunk < len) fetch(t0 + kChunk);
     }
-    __syncthreads();
     float k[DS], proj[kCols];
     {
       float pj[kCols] = {0.f, 0.f, 0.f, 0.f};
@@ -151,42 +235,74 @@ head_delta_kernel(HeadDelta a, SeqBatch s) {
     }
     const bool live = c0 < ncols;
     const int cl = live ? c0 : 0;                    // (lanes behind the last column compute on the first, and store nothing)
-    for (int tt = 0; tt < n; ++tt) {
-      const float g = sg[tt], beta = sbeta[tt];
-      const float4 v4 = *reinterpret_cast<const float4*>(sv + tt * cols + cl);
-      const float u[kCols] = {beta * (v4.x - g * proj[0]), beta * (v4.y - g * proj[1]), beta * (v4.z - g * proj[2]),
-                              beta * (v4.w - g * proj[3])};
-      float nm[kCols] = {0.f, 0.f, 0.f, 0.f}, pj[kCols] = {0.f, 0.f, 0.f, 0.f};
+    // a token's operands are in registers when its turn comes; the next token's are on their way (behind the pass's last row
+    // these reads meet LDS of other arrays, and what they return is never used)
+    struct Operands {
+      float q[DS], kn[DS];                           // its query, the NEXT token's key
+      float4 v;
+      float g, beta;
+    } cur, nxt;
+    auto read = [&](int tt, Operands& o) {
       const float* pq = sq + tt * KP + 4 * part;
-      const float* pk = sk + (tt + 1) * KP + 4 * part;      // the next token's key (row n: stale or unset, its sums unused)
+      const float* pk = sk + (tt + 1) * KP + 4 * part;
 #pragma unroll
       for (int ii = 0; ii < DS; ii += 4) {
         const float4 q4 = *reinterpret_cast<const float4*>(pq + SP * ii), n4 = *reinterpret_cast<const float4*>(pk + SP * ii);
-        const float qv[4] = {q4.x, q4.y, q4.z, q4.w}, nv[4] = {n4.x, n4.y, n4.z, n4.w};
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-#pragma unroll
-          for (int c = 0; c < kCols; ++c) {
-            const float x = g * S[c][ii + e] + k[ii + e] * u[c];
-            S[c][ii + e] = x;
-            nm[c] += x * qv[e];
-            pj[c] += x * nv[e];
-          }
-          k[ii + e] = nv[e];
-        }
+        o.q[ii] = q4.x, o.q[ii + 1] = q4.y, o.q[ii + 2] = q4.z, o.q[ii + 3] = q4.w;
+        o.kn[ii] = n4.x, o.kn[ii + 1] = n4.y, o.kn[ii + 2] = n4.z, o.kn[ii + 3] = n4.w;
       }
+      o.v = *reinterpret_cast<const float4*>(sv + tt * cols + cl);
+      o.g = sg[tt];
+      o.beta = sbeta[tt];
+    };
+    // S with the token that has key kt and operands o; its read-out to LDS, the next token's S^T kn to proj
+    auto token = [&](int tt, const float* kt, const Operands& o) {
+      const float u[kCols] = {o.beta * (o.v.x - o.g * proj[0]), o.beta * (o.v.y - o.g * proj[1]),
+                              o.beta * (o.v.z - o.g * proj[2]), o.beta * (o.v.w - o.g * proj[3])};
+      float nm[kCols] = {0.f, 0.f, 0.f, 0.f}, pj[kCols] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ii = 0; ii < DS; ++ii)
+#pragma unroll
+        for (int c = 0; c < kCols; ++c) {
+          const float x = o.g * S[c][ii] + kt[ii] * u[c];
+          S[c][ii] = x;
+          nm[c] += x * o.q[ii];
+          pj[c] += x * o.kn[ii];
+        }
 #pragma unroll
       for (int c = 0; c < kCols; ++c) {
         nm[c] = lanes_sum<SP>(nm[c]);
         proj[c] = lanes_sum<SP>(pj[c]);
       }
       if (live && part == 0) *reinterpret_cast<float4*>(so + tt * cols + c0) = float4{nm[0], nm[1], nm[2], nm[3]};
+    };
+    read(0, cur);
+    int tt = 0;
+    for (; tt + 2 <= n; tt += 2) {                   // two tokens per round: the operands change names, not registers
+      read(tt + 1, nxt);
+      token(tt, k, cur);
+      float kc[DS];
+#pragma unroll
+      for (int ii = 0; ii < DS; ++ii) kc[ii] = cur.kn[ii];
+      read(tt + 2, cur);
+      token(tt + 1, kc, nxt);
+#pragma unroll
+      for (int ii = 0; ii < DS; ++ii) k[ii] = nxt.kn[ii];
     }
+    if (tt < n) token(tt, k, cur);
     __syncthreads();
     if (a.raw) {                                     // the head's other columns are other workgroups': norm and gate follow
-      for (int e = j; e < n * ncols; e += NT) {
-        const int tt = e / ncols, i = e % ncols;
-        a.raw[(start + t0 + tt) * (int64_t)H * Dv + vc + i] = so[tt * cols + i];
+      for (int r = o_row; r < n; r += o_step) {
+        const float4 x = *reinterpret_cast<const float4*>(so + r * cols + o_col);
+        float* to = a.raw + (start + t0 + r) * (int64_t)H * Dv + vc + o_col;
+        if (quad) {
+          *reinterpret_cast<float4*>(to) = x;
+        } else {
+          const float xs[kCols] = {x.x, x.y, x.z, x.w};
+#pragma unroll
+          for (int c = 0; c < kCols; ++c)
+            if (o_col + c < ncols) to[c] = xs[c];
+        }
       }
       continue;
     }
@@ -251,8 +367,13 @@ static int launch_hd(const HeadDelta& a, const SeqBatch& s, int ranges, bool vec
   const unsigned threads = (unsigned)(((a.cols + kCols - 1) / kCols * SP + 63) / 64 * 64);
   const size_t lds = ((size_t)(2 * CH + 1) * KP + 2 * CH * a.cols + 3 * CH) * sizeof(float);
   static_assert(((2 * CH + 1) * KP + 2 * CH * kHdMaxV + 3 * CH) * sizeof(float) <= 64 * 1024, "LDS of the widest head");
-  if (vec) head_delta_kernel<Tag, KP, true><<<grid, threads, lds, st>>>(a, s);
-  else head_delta_kernel<Tag, KP, false><<<grid, threads, lds, st>>>(a, s);
+  if (threads <= 512) {          // (a larger workgroup leaves a lane half the registers)
+    if (vec) head_delta_kernel<Tag, KP, true, 512><<<grid, threads, lds, st>>>(a, s);
+    else head_delta_kernel<Tag, KP, false, 512><<<grid, threads, lds, st>>>(a, s);
+  } else {
+    if (vec) head_delta_kernel<Tag, KP, true, 1024><<<grid, threads, lds, st>>>(a, s);
+    else head_delta_kernel<Tag, KP, false, 1024><<<grid, threads, lds, st>>>(a, s);
+  }
   SP_LAUNCH_CHECK();
   if (a.raw) {
     const int64_t jobs = T * a.H;

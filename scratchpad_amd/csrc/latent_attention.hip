@@ -152,15 +152,16 @@ latent_attention_kernel(void* out, const void* q_lat, int64_t lat_token_stride, 
 
 // ---- the same attention on the matrix cores, for 16-bit types -------------------------------------------------------
 // All heads of a token read the same pool rows, so the queries of one request are ONE list of rows (token-major, then head)
-// whatever the head count.  A workgroup of 4 waves takes RB blocks of 16 such rows and walks the keys they can see in tiles
+// whatever the head count.  A workgroup of NW waves takes RB blocks of 16 such rows and walks the keys they can see in tiles
 // of 64, staged in LDS row by row (the next tile's rows are in flight during the work on this one):
 //   S^T = K Q^T   v_mfma_f32_16x16x32, first operand = 16 key rows from LDS, second = the query fragments, in registers for
-//                 the whole walk: wave w forms KBW of the tile's 4 key blocks for RBW of the RB row blocks.  A lane receives
-//                 four keys of ONE query; a query's maximum is a reduction over its lanes and, through LDS, over the waves.
+//                 the whole walk (rows too wide for that: the later steps' fragments wait in LDS): wave w forms KBW of the
+//                 tile's 4 key blocks for RBW of the RB row blocks.  A lane receives four keys of ONE query; a query's maximum is a reduction over its lanes and, through LDS, over the waves.
 //   P             exp of the scores, as a 16-bit value plus its 16-bit remainder (the weights are never rounded to 8 bits
 //                 of mantissa), goes to LDS in exactly the register layout the second product wants.
 //   O^T = V^T P^T the value is the first C columns of the same rows: its transposed fragments come from the key tile by
 //                 transposing LDS reads.  Wave w owns the value channels [16 DTW w, 16 DTW (w + 1)) of all RB row blocks.
+// Two waves per SIMD (NW = 8) where there are rows enough: one's softmax runs under the other's matrix instructions.
 // With splits > 1 the tiles of a row block are shared out over blockIdx.y; every share writes its unnormalised sum, maximum
 // and denominator, and latent_merge_kernel joins them in the order of the keys (decode steps: few rows, many keys).
 typedef float f32x4_l __attribute__((ext_vector_type(4)));
@@ -191,26 +192,34 @@ struct LatentArgs {
 };
 
 constexpr int kKeyTile = 64;
+constexpr float kSlack = 10.f;                       // in powers of two
 template <int KS>
 constexpr int key_row() { return 32 * KS + 8; }      // elements per LDS row: 16 bytes of padding spread the rows over the banks
 template <int KS, int RB>
+constexpr int query_steps() { return KS > 10 && RB > 1 ? (RB > 2 ? 4 : KS / 3) : KS; }      // steps whose query fragments stay in registers
+template <int KS, int RB, int NW>
 constexpr size_t latent_lds() {
-  return (size_t)kKeyTile * key_row<KS>() * 2 + (size_t)RB * 4096 + (4 * 2 * 16 + RB * 16 + 4 * 2 * 16) * sizeof(float);
+  return (size_t)kKeyTile * key_row<KS>() * 2 + (size_t)RB * 4096 + (size_t)RB * (KS - query_steps<KS, RB>()) * 1024 +
+         (NW * 2 * 16 + RB * 16 + NW * 2 * 16 + kKeyTile) * 4;
 }
 
-template <typename Tag, int KS, int DTW, int RB>
-__global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBatch s) {
+template <typename Tag, int KS, int DTW, int RB, int NW>
+__global__ void __launch_bounds__(64 * NW, NW / 4) latent_mfma_kernel(LatentArgs a, SeqBatch s) {
   typedef Elem<Tag> E;
   constexpr int RBW = RB > 1 ? 2 : 1;                 // row blocks a wave scores
   constexpr int GROUPS = RB / RBW;                    // groups of row blocks
-  constexpr int KBW = GROUPS;                         // key blocks (of 4) a wave scores: GROUPS * (4 / KBW) = 4 waves
+  constexpr int KBW = 4 * GROUPS / NW;                // key blocks (of 4) a wave scores: GROUPS * (4 / KBW) = NW waves
+  static_assert(KBW >= 1 && KBW * NW == 4 * GROUPS, "every key block of every row block has one wave");
   constexpr int KR = key_row<KS>();
   extern __shared__ __attribute__((aligned(16))) char lds[];
   uint16_t* sk = (uint16_t*)lds;                                       // [64][KR]
   u32x2* sp_ = (u32x2*)(lds + (size_t)kKeyTile * KR * 2);              // [RB][2][4 key blocks][64 lanes]
-  float* smax = (float*)(lds + (size_t)kKeyTile * KR * 2 + RB * 4096); // [4 waves][RBW][16]
-  float* scorr = smax + 4 * 2 * 16;                                    // [RB][16]
-  float* ssum = scorr + RB * 16;                                       // [4 waves][RBW][16]
+  constexpr int KQ = query_steps<KS, RB>();
+  u32x4* sqf = (u32x4*)(lds + (size_t)kKeyTile * KR * 2 + RB * 4096);  // [RB][KS - KQ][64 lanes]
+  float* smax = (float*)(sqf + RB * (KS - KQ) * 64);                   // [NW][RBW][16]
+  float* scorr = smax + NW * 2 * 16;                                   // [RB][16]
+  float* ssum = scorr + RB * 16;                                       // [NW][RBW][16]
+  int32_t* sslot = (int32_t*)(ssum + NW * 2 * 16);                     // [64] pool rows of the next tile's keys
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
   const int rg = wave % GROUPS, kg = wave / GROUPS;
   // which request and which of its row tiles
@@ -237,12 +246,13 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
   const int64_t last_row = row0 + 16 * RB <= rows ? row0 + 16 * RB - 1 : rows - 1;
   const int64_t keys = prefix + last_row / a.H + 1;
   const int64_t tiles_k = (keys + kKeyTile - 1) / kKeyTile;
+  const float scale2 = a.scale * 1.4426950408889634f;                  // scores in powers of two
   const int64_t per = (tiles_k + a.splits - 1) / a.splits;
   const int64_t kt0 = (int64_t)blockIdx.y * per, kt1 = kt0 + per < tiles_k ? kt0 + per : tiles_k;
   const int32_t* table = a.req_to_token + load_idx(s.req_pool_indices, b, s.idx64) * a.table_stride;
   const int chunks = (a.C + a.R) / 8;                                  // 16-byte pieces of a pool row
   // this lane's query rows (column r16 of every S^T block): fragments and the last key each may see
-  u32x4 qf[RBW][KS];
+  u32x4 qf[RBW][KQ];
   int64_t qpos[RBW];
 #pragma unroll
   for (int i = 0; i < RBW; ++i) {
@@ -256,13 +266,9 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
       u32x4 f = {0u, 0u, 0u, 0u};
       if (on && k < a.C) f = ld16((const char*)a.q_lat + (t * a.lat_token_stride + h * a.lat_head_stride + k) * 2);
       else if (on && k < a.C + a.R) f = ld16((const char*)a.q_rot + (t * a.qrot_token_stride + h * a.qrot_head_stride + k - a.C) * 2);
-      qf[i][st] = f;
+      if (st < KQ) qf[i][st < KQ ? st : 0] = f;
+      else if (kg == 0) sqf[((rg * RBW + i) * (KS - KQ) + st - KQ) * 64 + lane] = f;      // (read behind the walk's barriers)
     }
-  }
-  // columns behind the row are zero in every tile
-  for (int e = threadIdx.x; e < kKeyTile * (4 * KS - chunks); e += 256) {
-    const int n = 4 * KS - chunks, key = e / n, c = chunks + e % n;
-    st16((char*)(sk + key * KR + 8 * c), u32x4{0u, 0u, 0u, 0u});
   }
   f32x4_l oacc[DTW][RB];
 #pragma unroll
@@ -275,65 +281,93 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
     m[i] = -INFINITY;
     l[i] = 0.f;
   }
-  // 16-byte pieces this thread moves per tile: threadIdx.x + 256 u
-  const int dk = 256 / chunks, dc = 256 % chunks, key_first = threadIdx.x / chunks, c_first = threadIdx.x % chunks;
-  u32x4 stage[KS];
-  auto fetch = [&](int64_t kt) {
-    int key = key_first, c = c_first;
+  // a thread moves ONE 16-byte column of the rows key_first, key_first + KPP, ... of every tile: its addresses differ by
+  // constants.  Keys behind the last one and columns behind the row repeat the last of them - finite numbers that meet a zero
+  // weight or a zero of the query - so that no load waits for a branch
+  constexpr int CW = 4 * KS, KPP = 64 * NW / CW, NP = (kKeyTile + KPP - 1) / KPP;
+  const int key_first = threadIdx.x / CW, c = threadIdx.x % CW;
+  const bool mover = key_first < KPP;
+  const char* column = (const char*)a.pool + 16 * (c < chunks ? c : chunks - 1);
+  u32x4 stage[NP];
+  auto fetch = [&]() {                                                 // from the slots in LDS, behind a barrier
+    constexpr int PART = 6;                                            // addresses formed at a time
 #pragma unroll
-    for (int u = 0; u < KS; ++u) {
-      const int64_t kk = kt * kKeyTile + key;
-      stage[u] = u32x4{0u, 0u, 0u, 0u};
-      if (key < kKeyTile && kk < keys) stage[u] = ld16((const char*)a.pool + ((int64_t)table[kk] * a.pool_stride + 8 * c) * 2);
-      key += dk;
-      c += dc;
-      if (c >= chunks) {
-        c -= chunks;
-        ++key;
-      }
+    for (int u0 = 0; u0 < NP; u0 += PART) {
+      int32_t row[PART];
+#pragma unroll
+      for (int u = u0; u < NP && u < u0 + PART; ++u)
+        row[u - u0] = sslot[key_first + u * KPP < kKeyTile ? key_first + u * KPP : kKeyTile - 1];
+#pragma unroll
+      for (int u = u0; u < NP && u < u0 + PART; ++u) stage[u] = ld16(column + (int64_t)row[u - u0] * (2 * a.pool_stride));
+      __builtin_amdgcn_sched_barrier(0);
     }
   };
-  if (kt0 < kt1) fetch(kt0);
+  auto slot_of = [&](int64_t kt) {                                     // the slot of a tile's key (threads 0 .. 63 use it)
+    const int64_t kk = kt * kKeyTile + (threadIdx.x & 63);
+    return table[kk < keys ? kk : keys - 1];
+  };
+  int32_t slot = slot_of(kt0);
+  if (threadIdx.x < kKeyTile) sslot[threadIdx.x] = slot;
+  __syncthreads();
+  if (kt0 < kt1) fetch();
+  slot = slot_of(kt0 + 1);
   for (int64_t kt = kt0; kt < kt1; ++kt) {
     __syncthreads();                                                   // the previous tile's readers are done
-    {
-      int key = key_first, c = c_first;
+    if (mover) {
 #pragma unroll
-      for (int u = 0; u < KS; ++u) {
+      for (int u = 0; u < NP; ++u) {
+        const int key = key_first + u * KPP;
         if (key < kKeyTile) st16((char*)(sk + key * KR + 8 * c), stage[u]);
-        key += dk;
-        c += dc;
-        if (c >= chunks) {
-          c -= chunks;
-          ++key;
-        }
       }
     }
+    if (threadIdx.x < kKeyTile) sslot[threadIdx.x] = slot;
     __syncthreads();
-    if (kt + 1 < kt1) fetch(kt + 1);
+    if (kt + 1 < kt1) fetch();
+    slot = slot_of(kt + 2);
     f32x4_l sacc[RBW][KBW];
 #pragma unroll
     for (int i = 0; i < RBW; ++i)
 #pragma unroll
       for (int j = 0; j < KBW; ++j) sacc[i][j] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+    // key fragments two steps ahead of their use; the barriers to the scheduler keep it from loading them all at once
+    constexpr int AHEAD = 2;
+    u32x4 kf[AHEAD + 1][KBW];
+    u32x4 qs[AHEAD + 1][RBW];                                          // query fragments that wait in LDS
+    auto query_frag = [&](int st, int i) { return sqf[((rg * RBW + i) * (KS - KQ) + st - KQ) * 64 + lane]; };
+    auto key_frag = [&](int st, int j) { return ld16((const char*)(sk + (16 * (kg * KBW + j) + r16) * KR + 32 * st + 8 * qd)); };
 #pragma unroll
-    for (int st = 0; st < KS; ++st)
+    for (int st = 0; st < AHEAD && st < KS; ++st)
 #pragma unroll
-      for (int j = 0; j < KBW; ++j) {
-        const u32x4 kf = ld16((const char*)(sk + (16 * (kg * KBW + j) + r16) * KR + 32 * st + 8 * qd));
+      for (int j = 0; j < KBW; ++j) kf[st][j] = key_frag(st, j);
 #pragma unroll
-        for (int i = 0; i < RBW; ++i) sacc[i][j] = mfma_l<Tag>(kf, qf[i][st], sacc[i][j]);
+    for (int st = 0; st < KS; ++st) {
+      if (st + AHEAD < KS) {
+#pragma unroll
+        for (int j = 0; j < KBW; ++j) kf[(st + AHEAD) % (AHEAD + 1)][j] = key_frag(st + AHEAD, j);
+        if (st + AHEAD >= KQ)
+#pragma unroll
+          for (int i = 0; i < RBW; ++i) qs[(st + AHEAD) % (AHEAD + 1)][i] = query_frag(st + AHEAD, i);
       }
+#pragma unroll
+      for (int i = 0; i < RBW; ++i) {
+        const u32x4 q = st < KQ ? qf[i][st < KQ ? st : 0] : qs[st % (AHEAD + 1)][i];
+#pragma unroll
+        for (int j = 0; j < KBW; ++j) sacc[i][j] = mfma_l<Tag>(kf[st % (AHEAD + 1)][j], q, sacc[i][j]);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+    }
     float mx[RBW];
+    int edge[RBW];                                                     // the last key of this tile the query may see
 #pragma unroll
     for (int i = 0; i < RBW; ++i) {
+      const int64_t left = qpos[i] - kt * kKeyTile;
+      edge[i] = left < 0 ? -1 : (left > kKeyTile ? kKeyTile : (int)left);
       mx[i] = -INFINITY;
 #pragma unroll
       for (int j = 0; j < KBW; ++j)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int64_t kk = kt * kKeyTile + 16 * (kg * KBW + j) + 4 * qd + r;
-          const float v = kk <= qpos[i] ? sacc[i][j][r] * a.scale : -INFINITY;
+          const float v = 16 * (kg * KBW + j) + 4 * qd + r <= edge[i] ? sacc[i][j][r] * scale2 : -INFINITY;
           sacc[i][j][r] = v;
           mx[i] = fmaxf(mx[i], v);
         }
@@ -346,9 +380,12 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
     for (int i = 0; i < RBW; ++i) {
       float m_new = m[i];
 #pragma unroll
-      for (int w = rg; w < 4; w += GROUPS) m_new = fmaxf(m_new, smax[(w * RBW + i) * 16 + r16]);
+      for (int w = rg; w < NW; w += GROUPS) m_new = fmaxf(m_new, smax[(w * RBW + i) * 16 + r16]);
+      // the reference of the exponentials moves only when the maximum has left it by kSlack: sums stay far from overflow, and
+      // most tiles need no rescaling
+      if (m_new <= m[i] + kSlack) m_new = m[i];
       const float m_safe = m_new == -INFINITY ? 0.f : m_new;           // nothing seen yet: every weight is exp(-inf) = 0
-      const float corr = expf(m[i] - m_safe);
+      const float corr = m_new == m[i] ? 1.f : __builtin_amdgcn_exp2f(m[i] - m_safe);
       m[i] = m_new;
       float psum = 0.f;
 #pragma unroll
@@ -356,7 +393,7 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
         float p[8], rest[8], back[8];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          p[r] = expf(sacc[i][j][r] - m_safe);
+          p[r] = __builtin_amdgcn_exp2f(sacc[i][j][r] - m_safe);
           psum += p[r];
           p[4 + r] = 0.f;
         }
@@ -377,37 +414,44 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
 #pragma unroll
     for (int i = 0; i < RB; ++i) cr[i] = scorr[i * 16 + r16];
 #pragma unroll
-    for (int d = 0; d < DTW; ++d)
+    for (int i = 0; i < RB; ++i)
+      if (__any(cr[i] != 1.f)) {
+#pragma unroll
+        for (int d = 0; d < DTW; ++d)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) oacc[d][i][r] *= cr[i];
+      }
+#pragma unroll
+    for (int hh = 0; hh < 2; ++hh) {
+      u32x4 pw[2][RB];                                                 // the weights, their remainders
 #pragma unroll
       for (int i = 0; i < RB; ++i)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) oacc[d][i][r] *= cr[i];
-#pragma unroll
-    for (int hh = 0; hh < 2; ++hh) {
-      u32x4 ph[RB], pl[RB];
-#pragma unroll
-      for (int i = 0; i < RB; ++i) {
-        const u32x2* at = sp_ + (i * 8 + 2 * hh) * 64 + lane;
-        const u32x2 h0 = at[0], h1 = at[64], l0 = at[256], l1 = at[320];
-        ph[i] = u32x4{h0[0], h0[1], h1[0], h1[1]};
-        pl[i] = u32x4{l0[0], l0[1], l1[0], l1[1]};
-      }
-#pragma unroll
-      for (int d = 0; d < DTW; ++d) {
-        const int ch = 16 * (wave * DTW + d);
-        if (ch >= a.C) continue;                                       // (the same for the whole wave)
-        // lane i of a 16-lane group addresses row 4 qd + (i >> 2), elements 4 (i & 3) .. + 3, and receives column i
-        const uint16_t* vp = sk + (32 * hh + 4 * qd + (r16 >> 2)) * KR + ch + 4 * (r16 & 3);
+        for (int e = 0; e < 2; ++e) {
+          const u32x2* at = sp_ + (i * 8 + 4 * e + 2 * hh) * 64 + lane;
+          const u32x2 p0 = at[0], p1 = at[64];
+          pw[e][i] = u32x4{p0[0], p0[1], p1[0], p1[1]};
+        }
+      // lane i of a 16-lane group addresses row 4 qd + (i >> 2), elements 4 (i & 3) .. + 3, and receives column i.  Channels
+      // behind C (a wave's last tiles where C < 64 DTW) read the row's other columns; their sums are never stored.
+      auto value_frag = [&](int d) {
+        const uint16_t* vp = sk + (32 * hh + 4 * qd + (r16 >> 2)) * KR + 16 * (wave * DTW + d) + 4 * (r16 & 3);
         const u32x2 v0 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                                                        (__attribute__((address_space(3))) s16x4_l*)vp));
         const u32x2 v1 = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                                                        (__attribute__((address_space(3))) s16x4_l*)(vp + 16 * KR)));
-        const u32x4 vf = {v0[0], v0[1], v1[0], v1[1]};
+        return u32x4{v0[0], v0[1], v1[0], v1[1]};
+      };
+      u32x4 vf[2];
+      vf[0] = value_frag(0);
 #pragma unroll
-        for (int i = 0; i < RB; ++i) {
-          oacc[d][i] = mfma_l<Tag>(vf, ph[i], oacc[d][i]);
-          oacc[d][i] = mfma_l<Tag>(vf, pl[i], oacc[d][i]);
-        }
+      for (int d = 0; d < DTW; ++d) {
+        if (d + 1 < DTW) vf[(d + 1) & 1] = value_frag(d + 1);
+#pragma unroll
+        for (int e = 0; e < 2; ++e)
+#pragma unroll
+          for (int i = 0; i < RB; ++i) oacc[d][i] = mfma_l<Tag>(vf[d & 1], pw[e][i], oacc[d][i]);
+        __builtin_amdgcn_sched_barrier(0);
       }
     }
   }
@@ -424,7 +468,7 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
   for (int i = 0; i < RB; ++i) {
     float den = 0.f;
 #pragma unroll
-    for (int w = i / RBW; w < 4; w += GROUPS) den += ssum[(w * RBW + i % RBW) * 16 + r16];
+    for (int w = i / RBW; w < NW; w += GROUPS) den += ssum[(w * RBW + i % RBW) * 16 + r16];
     inv[i] = den;
   }
   if (a.splits > 1 && kg == 0 && qd == 0) {
@@ -435,7 +479,10 @@ __global__ void __launch_bounds__(256, 1) latent_mfma_kernel(LatentArgs a, SeqBa
       if (r < rows) {
         float* at = ml + ((int64_t)blockIdx.y * a.T * a.H + start * a.H + r) * 2;
         at[0] = m[i];
-        at[1] = inv[rg * RBW + i];
+        float den = inv[i];
+        const float other = inv[RB - RBW + i];
+        if (rg > 0) den = other;
+        at[1] = den;
       }
     }
   }
@@ -470,12 +517,12 @@ __global__ void __launch_bounds__(128) latent_merge_kernel(LatentArgs a) {
   float M = -INFINITY;
   for (int s = 0; s < a.splits; ++s) M = fmaxf(M, ml[((int64_t)s * n + r) * 2]);      // (a row has seen itself: M is finite)
   float den = 0.f;
-  for (int s = 0; s < a.splits; ++s) den += ml[((int64_t)s * n + r) * 2 + 1] * expf(ml[((int64_t)s * n + r) * 2] - M);
+  for (int s = 0; s < a.splits; ++s) den += ml[((int64_t)s * n + r) * 2 + 1] * exp2f(ml[((int64_t)s * n + r) * 2] - M);
   const float inv = 1.f / den;
   for (int c = 4 * threadIdx.x; c < a.C; c += 512) {
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     for (int s = 0; s < a.splits; ++s) {
-      const float w = expf(ml[((int64_t)s * n + r) * 2] - M);
+      const float w = exp2f(ml[((int64_t)s * n + r) * 2] - M);
       if (w == 0.f) continue;                                          // a share without keys has written no sum
       float f[4];
       unpack16<f32_tag>(ld16(a.part + ((int64_t)s * n + r) * a.C + c), f);
@@ -489,21 +536,22 @@ __global__ void __launch_bounds__(128) latent_merge_kernel(LatentArgs a) {
   }
 }
 
-template <typename Tag, int KS, int DTW, int RB>
+template <typename Tag, int KS, int DT, int RB, int NW>
 static int launch_latent_mfma(const LatentArgs& a, const SeqBatch& s, hipStream_t st) {
-  constexpr size_t lds = latent_lds<KS, RB>();
+  constexpr size_t lds = latent_lds<KS, RB, NW>();
+  constexpr int DTW = DT / NW;
   if (lds > 64 * 1024) {         // the limit is the device's: raised once per device of the process
     static PerDevice<int> raised;
     int ok = 0;
     raised.get(ok, [&](int) {
-      return hipFuncSetAttribute((const void*)latent_mfma_kernel<Tag, KS, DTW, RB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+      return hipFuncSetAttribute((const void*)latent_mfma_kernel<Tag, KS, DTW, RB, NW>, hipFuncAttributeMaxDynamicSharedMemorySize,
                                  (int)lds) == hipSuccess ? 1 : 0;
     });
     if (!ok) return SP_ERR_LAUNCH;
   }
   const int64_t blocks = s.extend_seq_lens ? (a.T * a.H + 16 * RB - 1) / (16 * RB) + s.B
                                            : (int64_t)s.B * ((a.H + 16 * RB - 1) / (16 * RB));
-  latent_mfma_kernel<Tag, KS, DTW, RB><<<dim3((unsigned)blocks, (unsigned)a.splits), 256, lds, st>>>(a, s);
+  latent_mfma_kernel<Tag, KS, DTW, RB, NW><<<dim3((unsigned)blocks, (unsigned)a.splits), 64 * NW, lds, st>>>(a, s);
   SP_LAUNCH_CHECK();
   if (a.splits > 1) {
     latent_merge_kernel<Tag><<<dim3((unsigned)(a.T * a.H)), 128, 0, st>>>(a);
@@ -511,28 +559,30 @@ static int launch_latent_mfma(const LatentArgs& a, const SeqBatch& s, hipStream_
   }
   return SP_OK;
 }
-template <typename Tag, int KS, int DTW>
+template <typename Tag, int KS, int DT>
 static int launch_latent_rows(const LatentArgs& a, const SeqBatch& s, hipStream_t st) {
   const int64_t rows = s.extend_seq_lens ? 64 : a.H;                   // rows a request brings in a decode step
-  if (rows <= 16) return launch_latent_mfma<Tag, KS, DTW, 1>(a, s, st);
-  if (rows <= 32) return launch_latent_mfma<Tag, KS, DTW, 2>(a, s, st);
-  return launch_latent_mfma<Tag, KS, DTW, 4>(a, s, st);
+  if (rows <= 16) return launch_latent_mfma<Tag, KS, DT, 1, 4>(a, s, st);
+  if (rows <= 32) return launch_latent_mfma<Tag, KS, DT, 2, 4>(a, s, st);
+  return launch_latent_mfma<Tag, KS, DT, 4, (KS > 5 ? 8 : 4)>(a, s, st);      // (narrow rows: more workgroups per CU instead)
 }
 template <typename Tag>
 static int launch_latent(const LatentArgs& a, const SeqBatch& s, hipStream_t st) {
-  if (a.C + a.R <= 160 && a.C <= 128) return launch_latent_rows<Tag, 5, 2>(a, s, st);
-  if (a.C + a.R <= 320 && a.C <= 256) return launch_latent_rows<Tag, 10, 4>(a, s, st);
-  if (a.C + a.R <= 576 && a.C <= 512) return launch_latent_rows<Tag, 18, 8>(a, s, st);
+  if (a.C + a.R <= 160 && a.C <= 128) return launch_latent_rows<Tag, 5, 8>(a, s, st);
+  if (a.C + a.R <= 320 && a.C <= 256) return launch_latent_rows<Tag, 10, 16>(a, s, st);
+  if (a.C + a.R <= 576 && a.C <= 512) return launch_latent_rows<Tag, 18, 32>(a, s, st);
   return SP_ERR_UNSUPPORTED;
 }
 
 // ---- out[t, h, n] = sum_k w[h, n, k] x[t, h, k]  (times sigmoid(gate[t, h N + n])) ---------------------------------------
 // 16-bit: a wave forms TT x NT tiles of 16 tokens x 16 outputs of one head, operands straight from memory (a head's matrix is
-// small and stays in the L2); TW of the 4 waves lie along the tokens, the others along the outputs.
+// small and stays in the L2); TW of the 4 waves lie along the tokens, the others along the outputs.  With four output tiles the
+// rows of w are dealt to them so that a lane ends with 16 neighbouring outputs of its token, its row's four lanes with 64.
 template <typename Tag, int TT, int NT, int TW>
 __global__ void __launch_bounds__(256)
 head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const void* x, int64_t x_stride, int64_t x_head,
                         const void* w, const void* gate, int64_t gate_stride, int64_t T, int N, int K) {
+  const bool whole = N % 8 == 0 && out_stride % 8 == 0 && out_head % 8 == 0 && ((uintptr_t)out & 15) == 0;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
   const int64_t h = blockIdx.z;
   const int64_t t0 = ((int64_t)blockIdx.x * TW + wave % TW) * (16 * TT);
@@ -546,7 +596,8 @@ head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const v
   }
 #pragma unroll
   for (int j = 0; j < NT; ++j) {
-    const int n = n0 + 16 * j + r16 < N ? n0 + 16 * j + r16 : N - 1;
+    int n = n0 + (NT == 4 ? 16 * (r16 >> 2) + 4 * j + (r16 & 3) : 16 * j + r16);
+    n = n < N ? n : N - 1;
     wp[j] = (const char*)w + ((h * N + n) * (int64_t)K + 8 * qd) * 2;
   }
   f32x4_l acc[TT][NT];
@@ -554,7 +605,7 @@ head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const v
   for (int i = 0; i < TT; ++i)
 #pragma unroll
     for (int j = 0; j < NT; ++j) acc[i][j] = f32x4_l{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+#pragma unroll 4
   for (int k = 0; k < K; k += 32) {
     const bool on = k + 8 * qd < K;                                    // K is a multiple of 8
     u32x4 xf[TT], wf[NT];
@@ -567,14 +618,15 @@ head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const v
 #pragma unroll
       for (int j = 0; j < NT; ++j) acc[i][j] = mfma_l<Tag>(wf[j], xf[i], acc[i][j]);
   }
-  // acc[i][j][r] = out[t0 + 16 i + r16][n0 + 16 j + 4 qd + r]; N is a multiple of 4
+  // acc[i][j][r] = out[t0 + 16 i + r16][n0 + 16 j + 4 qd + r], or [n0 + 16 qd + 4 j + r] with four tiles; N is a multiple of 4
 #pragma unroll
   for (int i = 0; i < TT; ++i) {
     const int64_t t = t0 + 16 * i + r16;
     if (t >= T) continue;
+    u32x2 half = {0u, 0u};
 #pragma unroll
     for (int j = 0; j < NT; ++j) {
-      const int n = n0 + 16 * j + 4 * qd;
+      const int n = n0 + (NT == 4 ? 16 * qd + 4 * j : 16 * j + 4 * qd);
       if (n >= N) continue;
       float f[8] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3], 0.f, 0.f, 0.f, 0.f};
       if (gate) {
@@ -585,7 +637,13 @@ head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const v
         for (int e = 0; e < 4; ++e) f[e] /= 1.f + expf(-g[e]);
       }
       const u32x4 pk = pack16<Tag>(f);
-      *(u32x2*)((char*)out + (t * out_stride + h * out_head + n) * 2) = u32x2{pk[0], pk[1]};
+      char* to = (char*)out + (t * out_stride + h * out_head + n) * 2;
+      if (NT == 4 && whole) {                                          // outputs in pairs of tiles: 16 bytes
+        if (j % 2 == 0) half = u32x2{pk[0], pk[1]};
+        else st16(to - 8, u32x4{half[0], half[1], pk[0], pk[1]});
+      } else {
+        *(u32x2*)to = u32x2{pk[0], pk[1]};
+      }
     }
   }
 }

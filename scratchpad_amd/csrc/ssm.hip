@@ -91,6 +91,61 @@ conv_silu_kernel(void* out, int64_t out_stride, const void* in, int64_t in_strid
 
 constexpr int kMaxTaps = 16;
 
+// The same on 16-byte pieces of rows, at most 4 taps: a thread keeps one piece's latest inputs in registers while it walks RUN
+// consecutive tokens of the step (a request's start inside the run re-reads them), so a row is read once, not once per tap.
+constexpr int kConvRun = 8;
+template <typename Tag, int TAPS>
+__global__ void __launch_bounds__(kBlock)
+conv_silu_run_kernel(void* out, int64_t out_stride, const void* in, int64_t in_stride, const float* w, const float* bias,
+                     const float* state, int64_t state_stride, SeqBatch s, int64_t T, int C) {
+  typedef Elem<Tag> E;
+  constexpr int V = E::kVec;
+  const int c = (blockIdx.y * kBlock + threadIdx.x) * V;
+  if (c >= C) return;
+  const int64_t t0 = (int64_t)blockIdx.x * kConvRun, t1 = t0 + kConvRun < T ? t0 + kConvRun : T;
+  float wt[TAPS][V], bs[V], past[TAPS][V];           // past[j]: the input TAPS - 1 - j rows back (the last one: this row's)
+#pragma unroll
+  for (int x = 0; x < V; ++x) {
+    bs[x] = bias ? bias[c + x] : 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[j][x] = w[(int64_t)(c + x) * TAPS + j];
+  }
+  int b = -1;
+  int64_t start = 0, prefix = 0;
+  for (int64_t t = t0; t < t1; ++t) {
+    int nb;
+    int64_t nstart, nprefix;
+    seq_of_token(s, t, nb, nstart, nprefix);
+    if (nb != b) {                                   // (also the run's first token)
+      b = nb, start = nstart, prefix = nprefix;
+      const float* st = state + load_idx(s.req_pool_indices, b, s.idx64) * state_stride;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int64_t r = t - (TAPS - 1) + j;
+        if (r >= start) {
+          unpack16<Tag>(ld16((const char*)in + (r * in_stride + c) * E::kBytes), past[j]);
+        } else {
+          const int64_t back = start - r;            // 1 .. TAPS - 1 rows before the step
+#pragma unroll
+          for (int x = 0; x < V; ++x) past[j][x] = prefix - back >= 0 ? st[(TAPS - 1 - back) * C + c + x] : 0.f;
+        }
+      }
+    }
+    unpack16<Tag>(ld16((const char*)in + (t * in_stride + c) * E::kBytes), past[TAPS - 1]);
+    float o[V];
+#pragma unroll
+    for (int x = 0; x < V; ++x) {
+      float acc = bs[x];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) acc += wt[j][x] * past[j][x];
+      o[x] = acc / (1.f + expf(-acc));
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) past[j][x] = past[j + 1][x];
+    }
+    st16((char*)out + (t * out_stride + c) * E::kBytes, pack16<Tag>(o));
+  }
+}
+
 template <typename Tag>
 __global__ void __launch_bounds__(kBlock)
 conv_state_kernel(float* state, int64_t state_stride, const void* in, int64_t in_stride, SeqBatch s, int C, int taps) {
@@ -112,6 +167,31 @@ conv_state_kernel(float* state, int64_t state_stride, const void* in, int64_t in
     fresh[k] = val;
   }
   for (int k = 0; k < keep; ++k) st[(int64_t)k * C + c] = fresh[k];
+}
+
+// a decode step's single row per request: output and the moved state in one launch (a thread owns a channel of a request)
+template <typename Tag>
+__global__ void __launch_bounds__(kBlock)
+conv_silu_step_kernel(void* out, int64_t out_stride, const void* in, int64_t in_stride, const float* w, const float* bias,
+                      float* state, int64_t state_stride, SeqBatch s, int C, int taps) {
+  typedef Elem<Tag> E;
+  const int b = blockIdx.x;
+  const int c = blockIdx.y * kBlock + threadIdx.x;
+  if (c >= C) return;
+  int64_t start, len, prefix;
+  seq_span(s, b, start, len, prefix);
+  float* st = state + load_idx(s.req_pool_indices, b, s.idx64) * state_stride;
+  const int keep = taps - 1;
+  float acc = bias ? bias[c] : 0.f;
+  for (int k = 0; k < keep; ++k) {
+    const float val = prefix - (keep - k) >= 0 ? st[(int64_t)k * C + c] : 0.f;
+    acc += w[(int64_t)c * taps + k] * val;
+    if (k > 0) st[(int64_t)(k - 1) * C + c] = val;
+  }
+  const float cur = E::load(in, (int64_t)b * in_stride + c);
+  acc += w[(int64_t)c * taps + keep] * cur;
+  if (keep > 0) st[(int64_t)(keep - 1) * C + c] = cur;
+  E::store(out, (int64_t)b * out_stride + c, acc / (1.f + expf(-acc)));
 }
 
 constexpr int kChunk = 16;      // tokens staged in LDS per pass
@@ -256,8 +336,28 @@ extern "C" int sp_causal_conv_silu(void* out, int64_t out_stride, const void* in
   SP_CHECK_ARG(extend_seq_lens || num_tokens == batch_size);
   SEQ_BATCH(s);
   const unsigned cb = (unsigned)((channels + kBlock - 1) / kBlock);
-  SP_DISPATCH_DTYPE(dtype, (conv_silu_kernel<Tag><<<dim3((unsigned)num_tokens, cb), kBlock, 0, (hipStream_t)stream>>>(
-                               out, out_stride, in, in_stride, weight, bias, state, state_stride, s, channels, taps)));
+  if (!extend_seq_lens) {
+    SP_DISPATCH_DTYPE(dtype, (conv_silu_step_kernel<Tag><<<dim3((unsigned)batch_size, cb), kBlock, 0, (hipStream_t)stream>>>(
+                                 out, out_stride, in, in_stride, weight, bias, state, state_stride, s, channels, taps)));
+    SP_LAUNCH_CHECK();
+    return SP_OK;
+  }
+  const int vecn = dtype == SP_F32 ? 4 : 8;
+  if (taps <= 4 && num_tokens > 64 && channels % vecn == 0 && in_stride % vecn == 0 && out_stride % vecn == 0 &&
+      (((uintptr_t)in | (uintptr_t)out) & 15) == 0) {
+    const dim3 grid((unsigned)((num_tokens + kConvRun - 1) / kConvRun), (unsigned)((channels / vecn + kBlock - 1) / kBlock));
+#define SP_CONV(TAPS)                                                                                                  \
+  SP_DISPATCH_DTYPE(dtype, (conv_silu_run_kernel<Tag, TAPS><<<grid, kBlock, 0, (hipStream_t)stream>>>(                  \
+                               out, out_stride, in, in_stride, weight, bias, state, state_stride, s, num_tokens, channels)))
+    if (taps == 1) SP_CONV(1);
+    else if (taps == 2) SP_CONV(2);
+    else if (taps == 3) SP_CONV(3);
+    else SP_CONV(4);
+#undef SP_CONV
+  } else {
+    SP_DISPATCH_DTYPE(dtype, (conv_silu_kernel<Tag><<<dim3((unsigned)num_tokens, cb), kBlock, 0, (hipStream_t)stream>>>(
+                                 out, out_stride, in, in_stride, weight, bias, state, state_stride, s, channels, taps)));
+  }
   SP_LAUNCH_CHECK();
   if (taps > 1) {      // after every reader of the old state (stream order)
     SP_DISPATCH_DTYPE(dtype, (conv_state_kernel<Tag><<<dim3((unsigned)batch_size, cb), kBlock, 0, (hipStream_t)stream>>>(
