@@ -455,9 +455,9 @@ class PostNorm(nn.Module):
 
     def forward(self, x: torch.Tensor, y, dtype: torch.dtype, want_lo: bool = True) -> Optional[torch.Tensor]:
         mix = {}
-        if isinstance(y, tuple) != (self.branch_weight is not None):
+        if (type(y) is tuple) != (self.branch_weight is not None):      # (a mixture's rows are a tuple of their own type)
             raise RuntimeError("PostNorm: built for another number of branches")
-        if isinstance(y, tuple):
+        if type(y) is tuple:
             y, b = y
             mix = dict(b=b, wa=self.branch_weight.data[0], wb=self.branch_weight.data[1])
         elif not isinstance(y, torch.Tensor):
