@@ -463,7 +463,7 @@ SP_API int sp_latent_kv_store(void* pool, int64_t pool_stride, const void* dkv, 
  * A token at position p of its request sees the request's positions 0 .. p through req_to_token.  rank <= 1024.
  * (ABI 15) matrix != 0: 16-bit types with rank and rot_dim multiples of 8, rank <= 512, rank + rot_dim <= 576 and 16-byte
  * aligned rows run on the matrix cores; splits > 1 then shares the keys of every query over that many workgroups, which join
- * through the workspace (fp32, splits * T * heads * (rank + 2) values).                                              */
+ * through the workspace (fp32, splits * T * heads * (rank + 2) values; splits <= 64).                                            */
 SP_API int sp_latent_attention(void* out, const void* q_lat, int64_t lat_token_stride, int64_t lat_head_stride,
                                const void* q_rot, const void* pool, int64_t pool_stride, const int32_t* req_to_token,
                                int64_t table_stride, int64_t num_tokens, int heads, int rank, int rot_dim,

@@ -192,6 +192,7 @@ struct LatentArgs {
 };
 
 constexpr int kKeyTile = 64;
+constexpr int kMaxSplits = 64;
 constexpr float kSlack = 10.f;                       // in powers of two
 template <int KS>
 constexpr int key_row() { return 32 * KS + 8; }      // elements per LDS row: 16 bytes of padding spread the rows over the banks
@@ -514,20 +515,37 @@ __global__ void __launch_bounds__(128) latent_merge_kernel(LatentArgs a) {
   typedef Elem<Tag> E;
   const int64_t r = blockIdx.x, n = a.T * a.H, t = r / a.H, h = r % a.H;
   const float* ml = a.part + (int64_t)a.splits * n * a.C;
-  float M = -INFINITY;
-  for (int s = 0; s < a.splits; ++s) M = fmaxf(M, ml[((int64_t)s * n + r) * 2]);      // (a row has seen itself: M is finite)
-  float den = 0.f;
-  for (int s = 0; s < a.splits; ++s) den += ml[((int64_t)s * n + r) * 2 + 1] * exp2f(ml[((int64_t)s * n + r) * 2] - M);
-  const float inv = 1.f / den;
+  __shared__ float weight[kMaxSplits];
+  __shared__ float total;
+  __shared__ int last;
+  if (threadIdx.x < 64) {                            // a wave: lane s holds share s
+    float m = -INFINITY, l = 0.f;
+    if ((int)threadIdx.x < a.splits) {
+      m = ml[((int64_t)threadIdx.x * n + r) * 2];
+      l = ml[((int64_t)threadIdx.x * n + r) * 2 + 1];
+    }
+    float M = m;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) M = fmaxf(M, __shfl_xor(M, off, 64));        // (a row has seen itself: M is finite)
+    const float w = exp2f(m - M), den = wave_sum(w * l);
+    weight[threadIdx.x] = w;
+    // shares are dealt from the first key on: all shares up to the last one that saw a key have written a sum
+    const unsigned long long seen = __ballot(w > 0.f);
+    if (threadIdx.x == 0) {
+      total = den;
+      last = 63 - __clzll(seen);
+    }
+  }
+  __syncthreads();
+  const float inv = 1.f / total;
   for (int c = 4 * threadIdx.x; c < a.C; c += 512) {
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < a.splits; ++s) {
-      const float w = exp2f(ml[((int64_t)s * n + r) * 2] - M);
-      if (w == 0.f) continue;                                          // a share without keys has written no sum
+#pragma unroll 8
+    for (int s = 0; s <= last; ++s) {
       float f[4];
       unpack16<f32_tag>(ld16(a.part + ((int64_t)s * n + r) * a.C + c), f);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) acc[e] += w * f[e];
+      for (int e = 0; e < 4; ++e) acc[e] += weight[s] * f[e];
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) acc[e] *= inv;
@@ -720,7 +738,7 @@ extern "C" int sp_latent_attention(void* out, const void* q_lat, int64_t lat_tok
       rank + rot_dim <= 576 && al16 && lat_token_stride % 8 == 0 && lat_head_stride % 8 == 0 && qrot_token_stride % 8 == 0 &&
       qrot_head_stride % 8 == 0 && pool_stride % 8 == 0) {
     if (splits < 1) splits = 1;
-    SP_CHECK_ARG(splits == 1 || (workspace && splits <= 65535));
+    SP_CHECK_ARG(splits == 1 || (workspace && splits <= kMaxSplits));
     if (splits > 1 && workspace_floats < (int64_t)splits * num_tokens * heads * (rank + 2)) return SP_ERR_WORKSPACE;
     const LatentArgs a{out, q_lat, q_rot, pool, req_to_token, workspace, lat_token_stride, lat_head_stride, qrot_token_stride,
                        qrot_head_stride, pool_stride, table_stride, num_tokens, heads, rank, rot_dim, splits, scale};

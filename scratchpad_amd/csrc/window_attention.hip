@@ -284,6 +284,7 @@ pool_blocks_kernel(void* kpooled, void* vpooled, const void* kpool, const void* 
 }
 
 constexpr int kMaxPerLane = 4;       // value width Dv <= 64 * kMaxPerLane
+constexpr int kRows = 8;             // value rows a wave has in flight
 
 template <typename Tag, bool VEC>
 __device__ __forceinline__ float dot_row(const float* sq, const void* base, int64_t at, int D) {
@@ -291,6 +292,7 @@ __device__ __forceinline__ float dot_row(const float* sq, const void* base, int6
   float d = 0.f;
   if (VEC) {
     constexpr int V = E::kVec;
+#pragma unroll 4
     for (int i = 0; i < D; i += V) {
       float f[V];
       unpack16<Tag>(ld16((const char*)base + (at + i) * E::kBytes), f);
@@ -306,7 +308,7 @@ __device__ __forceinline__ float dot_row(const float* sq, const void* base, int6
 // One workgroup of NW waves per (token, query head) - 4 for the rows of prompts, 16 for single decoded tokens, where the
 // rows are few and each is long.  The query's keys are numbered blocks first, then the window's tokens, in tiles of 64;
 // wave w takes tiles w, w + NW, ...: lane = key for the scores, lane = value channel for the
-// weighted sum (4 keys' rows in flight at a time); the waves' partial (maximum, sum, weighted values) meet in LDS.
+// weighted sum; the waves' partial (maximum, sum, weighted values) meet in LDS.
 // The order of every sum depends on the query's position only, never on the batch or on how the prompt was cut.
 template <typename Tag, bool VEC, bool SIG>
 __global__ void __launch_bounds__(1024)
@@ -345,11 +347,12 @@ window_attention_kernel(void* out, int64_t out_stride, const void* q, int64_t q_
   for (int64_t k0 = (int64_t)wave * 64; k0 < total; k0 += 64 * NW) {
     const int n = (int)(total - k0 < 64 ? total - k0 : 64);
     float sc = -INFINITY;
+    int32_t slot = 0;
     if (lane < n) {
       const int64_t kk = k0 + lane;
       const bool blk = kk < nb;
-      const int64_t row = blk ? table[kk * P + P - 1] : table[w0 + (kk - nb)];
-      sc = dot_row<Tag, VEC>(sq, blk ? kpooled : kpool, row * kp_stride + (int64_t)g * D, D);
+      slot = blk ? table[kk * P + P - 1] : table[w0 + (kk - nb)];
+      sc = dot_row<Tag, VEC>(sq, blk ? kpooled : kpool, (int64_t)slot * kp_stride + (int64_t)g * D, D);
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
     }
     if constexpr (SIG) {                                // every visible key on its own: no maximum, no denominator
@@ -369,39 +372,29 @@ window_attention_kernel(void* out, int64_t out_stride, const void* q, int64_t q_
 #pragma unroll
       for (int i = 0; i < kMaxPerLane; ++i) acc[i] *= corr;
     }
-    int j = 0;
-    for (; j + 4 <= n; j += 4) {
-      int64_t at[4];
-      const void* src[4];
+    // eight keys' rows in flight; the rows are what the lanes looked up for the scores.  Behind the last key its row comes again
+    // with a weight of zero
+    for (int j = 0; j < n; j += kRows) {
+      int64_t at[kRows];
+      const void* src[kRows];
+      float wt[kRows];
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const int64_t kk = k0 + j + u;
-        const bool blk = kk < nb;
-        at[u] = (int64_t)(blk ? table[kk * P + P - 1] : table[w0 + (kk - nb)]) * vp_stride + vcol;
-        src[u] = blk ? vpooled : vpool;
+      for (int u = 0; u < kRows; ++u) {
+        const int ju = j + u < n ? j + u : n - 1;
+        at[u] = (int64_t)__builtin_amdgcn_readlane(slot, ju) * vp_stride + vcol;
+        src[u] = k0 + ju < nb ? vpooled : vpool;
+        wt[u] = j + u < n ? sw[j + u] : 0.f;
       }
 #pragma unroll
       for (int i = 0; i < kMaxPerLane; ++i) {
         const int c = lane + 64 * i;
         if (c < Dv) {
-          const float v0 = E::load(src[0], at[0] + c), v1 = E::load(src[1], at[1] + c);
-          const float v2 = E::load(src[2], at[2] + c), v3 = E::load(src[3], at[3] + c);
-          acc[i] += sw[j] * v0;
-          acc[i] += sw[j + 1] * v1;
-          acc[i] += sw[j + 2] * v2;
-          acc[i] += sw[j + 3] * v3;
-        }
-      }
-    }
-    for (; j < n; ++j) {
-      const int64_t kk = k0 + j;
-      const bool blk = kk < nb;
-      const int64_t at = (int64_t)(blk ? table[kk * P + P - 1] : table[w0 + (kk - nb)]) * vp_stride + vcol;
-      const void* src = blk ? vpooled : vpool;
+          float v[kRows];
 #pragma unroll
-      for (int i = 0; i < kMaxPerLane; ++i) {
-        const int c = lane + 64 * i;
-        if (c < Dv) acc[i] += sw[j] * E::load(src, at + c);
+          for (int u = 0; u < kRows; ++u) v[u] = E::load(src[u], at[u] + c);
+#pragma unroll
+          for (int u = 0; u < kRows; ++u) acc[i] += wt[u] * v[u];
+        }
       }
     }
     __builtin_amdgcn_wave_barrier();
