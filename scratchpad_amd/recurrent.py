@@ -31,7 +31,7 @@ class WKVMixer(nn.Module):
         n = heads * dim
         f32 = dict(dtype=torch.float32)
         self.mu = nn.Parameter(torch.zeros(len(self.MIXES), width, **f32), requires_grad=False)
-        self.rkvg = nn.Parameter(torch.empty(4, n, width, dtype=dtype), requires_grad=False)
+        self.rkvg_t = nn.Parameter(torch.empty(4, width, n, dtype=dtype), requires_grad=False)     # as the product reads them
         self.w1 = nn.Parameter(torch.empty(decay_rank, width, dtype=dtype), requires_grad=False)
         self.w2t = nn.Parameter(torch.zeros(decay_rank, n, **f32), requires_grad=False)      # W_w2 transposed, fp32
         self.w0 = nn.Parameter(torch.zeros(n, **f32), requires_grad=False)
@@ -47,7 +47,7 @@ class WKVMixer(nn.Module):
         shift = states.shift_state(self.layer_id)
         mixes = _native.token_shift(x, self.mu.data, shift, seq, dtype)               # [5, T, W]
         _native.save_last_rows(shift, x, seq)                                         # after its only reader this step
-        rkvg = torch.bmm(mixes[:4], self.rkvg.transpose(1, 2))                        # [4, T, H * D]
+        rkvg = torch.bmm(mixes[:4], self.rkvg_t)                                      # [4, T, H * D]
         decay = _native.wkv_decay(_native.linear(mixes[4], self.w1), self.w2t.data, self.w0.data)
         o = _native.wkv_recurrence(rkvg[0], rkvg[1], rkvg[2], rkvg[3], decay, self.u.data, self.norm.data,
                                    states.matrix_state(self.layer_id), seq, self.heads, self.dim, self.eps)

@@ -229,7 +229,7 @@ class TizalornForCausalLM(nn.Module):
             put(layer.norm1.weight, take(f"{p}.norm1"))
             if layer.kind == "wkv":
                 put(mix.mu, torch.stack([take(f"{p}.mix.mu.{s}") for s in WKVMixer.MIXES]))
-                put(mix.rkvg, torch.stack([take(f"{p}.mix.{s}") for s in "rkvg"]))
+                put(mix.rkvg_t, torch.stack([take(f"{p}.mix.{s}").t() for s in "rkvg"]))
                 put(mix.w1, take(f"{p}.mix.w1"))
                 put(mix.w2t, take(f"{p}.mix.w2").t())
                 for name in ("w0", "u", "norm", "o"):
