@@ -593,60 +593,19 @@ static int launch_latent(const LatentArgs& a, const SeqBatch& s, hipStream_t st)
 }
 
 // ---- out[t, h, n] = sum_k w[h, n, k] x[t, h, k]  (times sigmoid(gate[t, h N + n])) ---------------------------------------
-// 16-bit: a wave forms TT x NT tiles of 16 tokens x 16 outputs of one head, operands straight from memory (a head's matrix is
-// small and stays in the L2); TW of the 4 waves lie along the tokens, the others along the outputs.  With four output tiles the
-// rows of w are dealt to them so that a lane ends with 16 neighbouring outputs of its token, its row's four lanes with 64.
-template <typename Tag, int TT, int NT, int TW>
-__global__ void __launch_bounds__(256)
-head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const void* x, int64_t x_stride, int64_t x_head,
-                        const void* w, const void* gate, int64_t gate_stride, int64_t T, int N, int K) {
+// acc[j][r] of a wave's 16 tokens = out[t + r16][n + 32 (j / 2) + 8 qd + 4 (j % 2) + r]: the output tiles come in pairs, to which
+// the rows of w are dealt so that a lane ends with 8 neighbouring outputs of its token (one 16-byte store).  N is a multiple of 4
+template <typename Tag, int NT>
+__device__ __forceinline__ void head_linear_store(const f32x4_l (&acc)[NT], void* out, int64_t out_stride, int64_t out_head,
+                                                  const void* gate, int64_t gate_stride, int64_t t, int n0, int64_t h, int N,
+                                                  int qd) {
   const bool whole = N % 8 == 0 && out_stride % 8 == 0 && out_head % 8 == 0 && ((uintptr_t)out & 15) == 0;
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
-  const int64_t h = blockIdx.z;
-  const int64_t t0 = ((int64_t)blockIdx.x * TW + wave % TW) * (16 * TT);
-  const int n0 = (blockIdx.y * (4 / TW) + wave / TW) * (16 * NT);
-  if (t0 >= T || n0 >= N) return;                                      // (no workgroup barrier below)
-  const char *xp[TT], *wp[NT];
-#pragma unroll
-  for (int i = 0; i < TT; ++i) {
-    const int64_t t = t0 + 16 * i + r16 < T ? t0 + 16 * i + r16 : T - 1;
-    xp[i] = (const char*)x + (t * x_stride + h * x_head + 8 * qd) * 2;
-  }
+  u32x2 half = {0u, 0u};
 #pragma unroll
   for (int j = 0; j < NT; ++j) {
-    int n = n0 + (NT == 4 ? 16 * (r16 >> 2) + 4 * j + (r16 & 3) : 16 * j + r16);
-    n = n < N ? n : N - 1;
-    wp[j] = (const char*)w + ((h * N + n) * (int64_t)K + 8 * qd) * 2;
-  }
-  f32x4_l acc[TT][NT];
-#pragma unroll
-  for (int i = 0; i < TT; ++i)
-#pragma unroll
-    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4_l{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k = 0; k < K; k += 32) {
-    const bool on = k + 8 * qd < K;                                    // K is a multiple of 8
-    u32x4 xf[TT], wf[NT];
-#pragma unroll
-    for (int i = 0; i < TT; ++i) xf[i] = on ? ld16(xp[i] + 2 * k) : u32x4{0u, 0u, 0u, 0u};
-#pragma unroll
-    for (int j = 0; j < NT; ++j) wf[j] = on ? ld16(wp[j] + 2 * k) : u32x4{0u, 0u, 0u, 0u};
-#pragma unroll
-    for (int i = 0; i < TT; ++i)
-#pragma unroll
-      for (int j = 0; j < NT; ++j) acc[i][j] = mfma_l<Tag>(wf[j], xf[i], acc[i][j]);
-  }
-  // acc[i][j][r] = out[t0 + 16 i + r16][n0 + 16 j + 4 qd + r], or [n0 + 16 qd + 4 j + r] with four tiles; N is a multiple of 4
-#pragma unroll
-  for (int i = 0; i < TT; ++i) {
-    const int64_t t = t0 + 16 * i + r16;
-    if (t >= T) continue;
-    u32x2 half = {0u, 0u};
-#pragma unroll
-    for (int j = 0; j < NT; ++j) {
-      const int n = n0 + (NT == 4 ? 16 * qd + 4 * j : 16 * j + 4 * qd);
-      if (n >= N) continue;
-      float f[8] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3], 0.f, 0.f, 0.f, 0.f};
+    const int n = n0 + (NT % 2 == 0 ? 32 * (j >> 1) + 8 * qd + 4 * (j & 1) : 16 * j + 4 * qd);
+    if (n < N) {
+      float f[8] = {acc[j][0], acc[j][1], acc[j][2], acc[j][3], 0.f, 0.f, 0.f, 0.f};
       if (gate) {
         float g[8];
         const u32x2 g2 = *(const u32x2*)((const char*)gate + (t * gate_stride + h * N + n) * 2);
@@ -656,13 +615,115 @@ head_linear_mfma_kernel(void* out, int64_t out_stride, int64_t out_head, const v
       }
       const u32x4 pk = pack16<Tag>(f);
       char* to = (char*)out + (t * out_stride + h * out_head + n) * 2;
-      if (NT == 4 && whole) {                                          // outputs in pairs of tiles: 16 bytes
+      if (NT % 2 == 0 && whole) {
         if (j % 2 == 0) half = u32x2{pk[0], pk[1]};
         else st16(to - 8, u32x4{half[0], half[1], pk[0], pk[1]});
       } else {
         *(u32x2*)to = u32x2{pk[0], pk[1]};
       }
     }
+  }
+}
+
+// Few tokens (16-bit): a wave per 16 tokens x 16 outputs of a head, operands straight from memory.
+template <typename Tag>
+__global__ void __launch_bounds__(256)
+head_linear_rows_kernel(void* out, int64_t out_stride, int64_t out_head, const void* x, int64_t x_stride, int64_t x_head,
+                        const void* w, const void* gate, int64_t gate_stride, int64_t T, int N, int K) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
+  const int64_t h = blockIdx.z, t0 = (int64_t)blockIdx.x * 16;
+  const int n0 = (blockIdx.y * 4 + wave) * 16;
+  if (n0 >= N) return;                                                 // (no workgroup barrier below)
+  const int64_t t = t0 + r16 < T ? t0 + r16 : T - 1;
+  const int n = n0 + r16 < N ? n0 + r16 : N - 1;
+  const char* xp = (const char*)x + (t * x_stride + h * x_head + 8 * qd) * 2;
+  const char* wp = (const char*)w + ((h * N + n) * (int64_t)K + 8 * qd) * 2;
+  f32x4_l acc[1] = {f32x4_l{0.f, 0.f, 0.f, 0.f}};
+  const int whole_k = K / 32 * 32;
+#pragma unroll 4
+  for (int k = 0; k < whole_k; k += 32) acc[0] = mfma_l<Tag>(ld16(wp + 2 * k), ld16(xp + 2 * k), acc[0]);
+  if (whole_k < K) {                                                   // K is a multiple of 8: the lanes behind it bring zeros
+    const bool on = whole_k + 8 * qd < K;
+    const u32x4 zero = {0u, 0u, 0u, 0u};
+    acc[0] = mfma_l<Tag>(on ? ld16(wp + 2 * whole_k) : zero, on ? ld16(xp + 2 * whole_k) : zero, acc[0]);
+  }
+  if (t0 + r16 < T) head_linear_store<Tag, 1>(acc, out, out_stride, out_head, gate, gate_stride, t0 + r16, n0, h, N, qd);
+}
+
+// Many tokens (16-bit): 128 tokens x TN outputs of a head per workgroup, both operands staged in LDS 64 columns at a time (whole
+// 128-byte lines per 8 lanes; an operand fragment taken straight from memory touches 16 lines per 16 lanes), the next columns in
+// flight during the products.  TN = 128: the 4 waves form 64 x 64 each; TN = 64: 32 x 64.
+constexpr int kHeadRow = 72;                                           // 64 columns + 16 bytes that spread the rows over the banks
+template <typename Tag, int TN>
+__global__ void __launch_bounds__(256)
+head_linear_tile_kernel(void* out, int64_t out_stride, int64_t out_head, const void* x, int64_t x_stride, int64_t x_head,
+                        const void* w, const void* gate, int64_t gate_stride, int64_t T, int N, int K) {
+  constexpr int WN = TN / 64, WT = 4 / WN, TT = 8 / WT, NT = 4, XP = 4, WP = TN / 32;
+  __shared__ __attribute__((aligned(16))) uint16_t sx[128 * kHeadRow], sw[TN * kHeadRow];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
+  const int64_t h = blockIdx.z, t0 = (int64_t)blockIdx.x * 128;
+  const int n0 = blockIdx.y * TN, row = threadIdx.x >> 3, col = 8 * (threadIdx.x & 7);
+  const char *xp[XP], *wp[WP];
+  int xl[XP], wl[WP];                                                  // where a piece lies in LDS
+#pragma unroll
+  for (int u = 0; u < XP; ++u) {
+    const int r = row + 32 * u;
+    xp[u] = (const char*)x + ((t0 + r < T ? t0 + r : T - 1) * x_stride + h * x_head) * 2;
+    xl[u] = r * kHeadRow + col;
+  }
+#pragma unroll
+  for (int u = 0; u < WP; ++u) {
+    const int r = row + 32 * u, m = r & 63;                            // output r of the tile -> row 16 j + r16 of its group of 64
+    wp[u] = (const char*)w + (h * N + (n0 + r < N ? n0 + r : N - 1)) * (int64_t)K * 2;
+    wl[u] = ((r & 64) + 16 * (2 * (m >> 5) + ((m >> 2) & 1)) + 4 * ((m >> 3) & 3) + (m & 3)) * kHeadRow + col;
+  }
+  u32x4 fx[XP], fw[WP];
+  auto fetch = [&](int k0) {                                           // columns behind K: the last ones again, as zeros
+    const int k = k0 + col, kc = 2 * (k < K ? k : K - 8);
+    const uint32_t keep = k < K ? 0xffffffffu : 0u;
+#pragma unroll
+    for (int u = 0; u < XP; ++u) fx[u] = ld16(xp[u] + kc);
+#pragma unroll
+    for (int u = 0; u < WP; ++u) fw[u] = ld16(wp[u] + kc);
+    if (k0 + 64 > K) {
+#pragma unroll
+      for (int u = 0; u < XP; ++u) fx[u] &= keep;
+#pragma unroll
+      for (int u = 0; u < WP; ++u) fw[u] &= keep;
+    }
+  };
+  f32x4_l acc[TT][NT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4_l{0.f, 0.f, 0.f, 0.f};
+  const int tw = (wave / WN) * 16 * TT, nw = (wave % WN) * 64;         // this wave's corner of the tile
+  fetch(0);
+  for (int k0 = 0; k0 < K; k0 += 64) {
+    __syncthreads();                                                   // the previous columns' readers are done
+#pragma unroll
+    for (int u = 0; u < XP; ++u) st16(sx + xl[u], fx[u]);
+#pragma unroll
+    for (int u = 0; u < WP; ++u) st16(sw + wl[u], fw[u]);
+    __syncthreads();
+    if (k0 + 64 < K) fetch(k0 + 64);
+#pragma unroll
+    for (int st = 0; st < 2; ++st) {
+      u32x4 xf[TT], wf[NT];
+#pragma unroll
+      for (int i = 0; i < TT; ++i) xf[i] = ld16(sx + (tw + 16 * i + r16) * kHeadRow + 32 * st + 8 * qd);
+#pragma unroll
+      for (int j = 0; j < NT; ++j) wf[j] = ld16(sw + (nw + 16 * j + r16) * kHeadRow + 32 * st + 8 * qd);
+#pragma unroll
+      for (int i = 0; i < TT; ++i)
+#pragma unroll
+        for (int j = 0; j < NT; ++j) acc[i][j] = mfma_l<Tag>(wf[j], xf[i], acc[i][j]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    const int64_t t = t0 + tw + 16 * i + r16;
+    if (t < T) head_linear_store<Tag, NT>(acc[i], out, out_stride, out_head, gate, gate_stride, t, n0 + nw, h, N, qd);
   }
 }
 
@@ -769,18 +830,18 @@ extern "C" int sp_head_linear(void* out, int64_t out_stride, int64_t out_head_st
                   out_head_stride % 4 == 0 && (!gate || gate_stride % 4 == 0);
   hipStream_t st = (hipStream_t)stream;
   if (al && (dtype == SP_BF16 || dtype == SP_F16)) {
-#define SP_HL(Tag, TT, NT, TW)                                                                                          \
-  head_linear_mfma_kernel<Tag, TT, NT, TW><<<dim3((unsigned)((num_tokens + 16 * TT * TW - 1) / (16 * TT * TW)),            \
-                                                  (unsigned)((n + 16 * NT * (4 / TW) - 1) / (16 * NT * (4 / TW))),        \
-                                                  (unsigned)heads), 256, 0, st>>>(                                        \
-      out, out_stride, out_head_stride, x, x_stride, x_head_stride, w, gate, gate_stride, num_tokens, n, k)
-    if (num_tokens <= 64) {
-      if (dtype == SP_BF16) SP_HL(bf16_tag, 1, 1, 1);
-      else SP_HL(f16_tag, 1, 1, 1);
-    } else {
-      if (dtype == SP_BF16) SP_HL(bf16_tag, 2, 4, 4);
-      else SP_HL(f16_tag, 2, 4, 4);
-    }
+#define SP_HL(KERNEL, TILE_T, TILE_N)                                                                                   \
+  KERNEL<<<dim3((unsigned)((num_tokens + TILE_T - 1) / TILE_T), (unsigned)((n + TILE_N - 1) / TILE_N), (unsigned)heads), 256, 0, \
+           st>>>(out, out_stride, out_head_stride, x, x_stride, x_head_stride, w, gate, gate_stride, num_tokens, n, k)
+#define SP_HL_TYPES(TILE_T, TILE_N, NAME, ...)                                     \
+  do {                                                                             \
+    if (dtype == SP_BF16) SP_HL((NAME<bf16_tag __VA_ARGS__>), TILE_T, TILE_N);     \
+    else SP_HL((NAME<f16_tag __VA_ARGS__>), TILE_T, TILE_N);                       \
+  } while (0)
+    if (num_tokens <= 64) SP_HL_TYPES(16, 64, head_linear_rows_kernel);
+    else if (n > 64) SP_HL_TYPES(128, 128, head_linear_tile_kernel, , 128);
+    else SP_HL_TYPES(128, 64, head_linear_tile_kernel, , 64);
+#undef SP_HL_TYPES
 #undef SP_HL
     SP_LAUNCH_CHECK();
     return SP_OK;
