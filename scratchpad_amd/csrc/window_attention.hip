@@ -441,10 +441,10 @@ window_attention_kernel(void* out, int64_t out_stride, const void* q, int64_t q_
 // One workgroup per (16 consecutive tokens of one request's portion, key/value head); wave w works for the group's query
 // head w (w + 4, ... in further passes).  Keys of the 16 queries' UNION (blocks up to the last query's, tokens from the
 // first query's window start to the last query) go by in tiles of 64; who sees what is a mask per (key, query).
-//   S^T = K Q^T   v_mfma_f32_16x16x32: first operand = 16 key rows straight from the pool (16 bytes per lane), second =
-//                 the query fragment held in registers; a lane receives S^T[key 4q + r][query r16]: four keys of ONE query,
+//   S^T = K Q^T   v_mfma_f32_16x16x32: first operand = 16 key rows from LDS (a fragment taken straight from the pool would
+//                 touch 16 lines per 16 lanes), second = the query fragment held in registers; a lane receives S^T[key 4q + r][query r16]: four keys of ONE query,
 //                 so the softmax of a query is a reduction over r, the tile's four key groups and the lanes q = 0..3.
-//   O^T = V^T P^T first operand = V^T from an LDS tile written transposed ([value channel][key], keys contiguous), second =
+//   O^T = V^T P^T first operand = V^T by transposing reads of the value rows in LDS, second =
 //                 P^T - exactly the registers the lane already holds: the key order inside a step of 32 is (4q .. 4q + 3 of
 //                 the first 16 keys, then of the second 16) for both operands, so P needs no exchange between lanes.
 // Scores, softmax and O are fp32; P enters the second product as a 16-bit value plus its 16-bit remainder (two products).
@@ -462,7 +462,7 @@ __device__ __forceinline__ f32x4_w mfma_w<f16_tag>(const u32x4& a, const u32x4& 
   return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8_w, a), __builtin_bit_cast(f16x8_w, b), c, 0, 0, 0);
 }
 
-constexpr int kVtRow = 72;      // 64 keys + 8 of padding per value channel (16-bit elements)
+typedef short s16x4_w __attribute__((ext_vector_type(4)));
 
 template <typename Tag, int DS, int DT, bool SIG>      // DS = dim / 32, DT = vdim / 16
 __global__ void __launch_bounds__(256)
@@ -472,8 +472,10 @@ window_attention_mfma_kernel(void* out, int64_t out_stride, const void* q, int64
                              int64_t lead, float scale, const float* sinks, float softcap, const float* head_bias, const void* gate,
                              int64_t gate_stride) {
   constexpr int D = 32 * DS, Dv = 16 * DT;
-  __shared__ uint16_t vt[Dv][kVtRow];
-  __shared__ int32_t sslot[64];
+  constexpr int KR = D + 8, VR = Dv + 8;                 // elements per LDS row: 16 bytes of padding spread the rows over the banks
+  constexpr int KP = D / 32, VP = Dv / 32;               // 16-byte pieces of a key (value) tile per thread
+  __shared__ __attribute__((aligned(16))) uint16_t skey[64 * KR], sval[64 * VR];
+  __shared__ int32_t sslot[64];                          // pool rows of the next tile's keys
   // which request and which of its 16-row tiles
   int tile = blockIdx.x, b = 0;
   for (; b < s.B; ++b) {
@@ -513,43 +515,57 @@ window_attention_mfma_kernel(void* out, int64_t out_stride, const void* q, int64
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) oacc[dt] = f32x4_w{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.f;
+    // the tiles go through registers, one ahead of the work; keys behind the last one repeat it, unseen by every query
+    auto entry = [&](int64_t k0, int key) { return k0 + key < totalU ? k0 + key : totalU - 1; };
+    auto slot_of = [&](int64_t k0) {                     // (threads 0 .. 63 use it)
+      const int64_t kk = entry(k0, threadIdx.x & 63);
+      return kk < nbU ? table[kk * P + P - 1] : table[w0U + (kk - nbU)];
+    };
+    u32x4 kst[KP], vst[VP];
+    auto fetch = [&](int64_t k0) {
+#pragma unroll
+      for (int u = 0; u < KP; ++u) {
+        const int c = threadIdx.x + 256 * u, key = c / (D / 8), col = c % (D / 8);
+        const void* src = entry(k0, key) < nbU ? kpooled : kpool;
+        kst[u] = ld16((const char*)src + ((int64_t)sslot[key] * kp_stride + (int64_t)g * D + 8 * col) * 2);
+      }
+#pragma unroll
+      for (int u = 0; u < VP; ++u) {
+        const int c = threadIdx.x + 256 * u, key = c / (Dv / 8), col = c % (Dv / 8);
+        const void* src = entry(k0, key) < nbU ? vpooled : vpool;
+        vst[u] = ld16((const char*)src + ((int64_t)sslot[key] * vp_stride + (int64_t)g * Dv + 8 * col) * 2);
+      }
+    };
+    int32_t slot = slot_of(0);
+    __syncthreads();                                     // (a further pass of heads: the last tile's readers are done)
+    if (threadIdx.x < 64) sslot[threadIdx.x] = slot;
+    __syncthreads();
+    fetch(0);
+    slot = slot_of(64);
     for (int64_t k0 = 0; k0 < totalU; k0 += 64) {
       __syncthreads();                                   // the previous tile's readers are done
-      if (threadIdx.x < 64) {
-        const int64_t kk = k0 + threadIdx.x;
-        int32_t sl = 0;
-        if (kk < totalU) sl = kk < nbU ? table[kk * P + P - 1] : table[w0U + (kk - nbU)];
-        sslot[threadIdx.x] = sl;
-      }
-      __syncthreads();
-      // V^T tile: thread = (key, 8 value channels); neighbouring lanes take neighbouring keys (conflict-free 2-byte writes)
-      for (int c = threadIdx.x; c < 64 * (Dv / 8); c += 256) {
-        const int key = c & 63, dvc = c >> 6;
-        const int64_t kk = k0 + key;
-        u32x4 val = {0u, 0u, 0u, 0u};
-        if (kk < totalU)
-          val = ld16((const char*)(kk < nbU ? vpooled : vpool) + ((int64_t)sslot[key] * vp_stride + (int64_t)g * Dv + 8 * dvc) * 2);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const uint32_t w2 = e == 0 ? val[0] : (e == 1 ? val[1] : (e == 2 ? val[2] : val[3]));
-          vt[8 * dvc + 2 * e][key] = (uint16_t)(w2 & 0xffffu);
-          vt[8 * dvc + 2 * e + 1][key] = (uint16_t)(w2 >> 16);
-        }
+      for (int u = 0; u < KP; ++u) {
+        const int c = threadIdx.x + 256 * u;
+        st16(skey + (c / (D / 8)) * KR + 8 * (c % (D / 8)), kst[u]);
       }
+#pragma unroll
+      for (int u = 0; u < VP; ++u) {
+        const int c = threadIdx.x + 256 * u;
+        st16(sval + (c / (Dv / 8)) * VR + 8 * (c % (Dv / 8)), vst[u]);
+      }
+      if (threadIdx.x < 64) sslot[threadIdx.x] = slot;
       __syncthreads();
+      if (k0 + 64 < totalU) fetch(k0 + 64);
+      slot = slot_of(k0 + 128);
       if (work) {
         f32x4_w sacc[4];
 #pragma unroll
         for (int sb = 0; sb < 4; ++sb) {
           sacc[sb] = f32x4_w{0.f, 0.f, 0.f, 0.f};
-          const int64_t kk = k0 + 16 * sb + r16;         // the key row this lane feeds
-          const bool kvalid = kk < totalU;
-          const char* kp = (const char*)(kk < nbU ? kpooled : kpool) + ((int64_t)sslot[16 * sb + r16] * kp_stride + (int64_t)g * D + 8 * qd) * 2;
 #pragma unroll
-          for (int st = 0; st < DS; ++st) {
-            const u32x4 a = kvalid ? ld16(kp + 64 * st) : u32x4{0u, 0u, 0u, 0u};
-            sacc[sb] = mfma_w<Tag>(a, qf[st], sacc[sb]);
-          }
+          for (int st = 0; st < DS; ++st)
+            sacc[sb] = mfma_w<Tag>(ld16(skey + (16 * sb + r16) * KR + 32 * st + 8 * qd), qf[st], sacc[sb]);
         }
         float mx = -INFINITY;
 #pragma unroll
@@ -614,8 +630,12 @@ window_attention_mfma_kernel(void* out, int64_t out_stride, const void* q, int64
 #pragma unroll
               for (int r = 0; r < 4; ++r) oacc[dt][r] *= corr;
             }
-            const u32x2 lo = *(const u32x2*)&vt[16 * dt + r16][32 * hh + 4 * qd];
-            const u32x2 hi = *(const u32x2*)&vt[16 * dt + r16][32 * hh + 16 + 4 * qd];
+            // lane i of a 16-lane group addresses row 4 qd + (i >> 2), elements 4 (i & 3) .. + 3, and receives column i
+            const uint16_t* vp = sval + (32 * hh + 4 * qd + (r16 >> 2)) * VR + 16 * dt + 4 * (r16 & 3);
+            const u32x2 lo = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                                                           (__attribute__((address_space(3))) s16x4_w*)vp));
+            const u32x2 hi = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                                                           (__attribute__((address_space(3))) s16x4_w*)(vp + 16 * VR)));
             const u32x4 a = {lo[0], lo[1], hi[0], hi[1]};
             oacc[dt] = mfma_w<Tag>(a, pb, oacc[dt]);
             oacc[dt] = mfma_w<Tag>(a, pr, oacc[dt]);
