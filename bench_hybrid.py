@@ -203,6 +203,11 @@ def instrument(clock: KernelClock, cfg):
         outs = out if isinstance(out, (tuple, list)) else (out,)
         return _nbytes(*a, *k.values(), *outs), 0, MATRIX
 
+    def embed(a, k, out):        # the rows gathered from the table(s), the results; not the whole tables
+        outs = out if isinstance(out, (tuple, list)) else (out,)
+        tables = 1 + (k.get("table") is not None)
+        return tables * outs[0].numel() * a[0].element_size() + _nbytes(*outs), 0, MATRIX
+
     def gemm(a, k, out):
         x, w = a[0], a[1]
         return _nbytes(x, w, out), 2 * x.shape[0] * w.shape[0] * w.shape[1], MATRIX
@@ -293,7 +298,7 @@ def instrument(clock: KernelClock, cfg):
              "latent_attention": latent, "moe_route": io, "moe_align": io, "moe_grouped_gemm": grouped, "moe_glu": io,
              "moe_combine": io, "rmsnorm": io, "fused_add_rmsnorm": io, "silu_and_mul": io, "rotary_embedding": io,
              "extend_attention": llama_extend, "decode_attention": llama_extend, "linear": gemm,
-             "embed_scale": io, "norm_shift": io, "stream_add": io, "qkv_rotary_store": io, "pool_blocks": io,
+             "embed_scale": embed, "norm_shift": io, "stream_add": io, "qkv_rotary_store": io, "pool_blocks": io,
              "window_attention": window, "small_linear_f32": small, "causal_conv_silu": io, "mamba2_scan": scan,
              "gated_group_norm": io, "mlstm_scan": mlstm, "moe_route_softmax": io,
              "gated_add_norm": io, "relu_square": io, "scale_softcap": io, "delta_gates": io, "delta_recurrence": delta,
